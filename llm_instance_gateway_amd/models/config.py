@@ -21,8 +21,9 @@ class LayerSpec:
     vector), the mixer's sizes and constants, and its feed-forward (None for
     a layer without one).  'latent_attention' keeps one paged row per token
     (the normalised key/value latent followed by the shared rotated key
-    part).  'wkv' keeps a matrix state per head and the previous token's
-    input row; 'parallel' keeps paged K/V for its attention branch and a
+    part), or nothing when it reads another layer's rows ('kv_from').  'wkv' keeps a matrix state per head and the previous token's
+    input row; 'retention' and 'mlstm' keep a matrix state per head (the
+    latter with a normaliser vector and a running maximum); 'parallel' keeps paged K/V for its attention branch and a
     matrix state per head for its recurrent branch.  `shift` says the mixer's input is blended with the previous
     token's, which costs one fp32 row of model width per sequence."""
 
@@ -79,6 +80,11 @@ class ModelConfig:
     # one stream without them is the ordinary residual.
     residual_streams: int = 1
     hyper_connections: bool = False
+    # Factor on the embedding rows.
+    embed_scale: float = 1.0
+    # Entries per layer of a second token table whose row enters the residual
+    # after every layer (0 = no such table).
+    token_side_dim: int = 0
 
     @property
     def is_moe(self) -> bool:
@@ -109,7 +115,7 @@ class ModelConfig:
             s = self.layer_specs[i]
             if s.type in ("attention", "attention_2"):
                 total += (s.mixer["kv_heads"] // tp_size) * (s.mixer["dim"] + s.mixer["vdim"])
-            elif s.type == "latent_attention":
+            elif s.type == "latent_attention" and s.mixer.get("kv_from") is None:
                 total += s.mixer["kv_rank"] + s.mixer["rot_dim"]
             elif s.type == "parallel":
                 # the attention branch caches normed keys and, as values, the
@@ -130,6 +136,11 @@ class ModelConfig:
             elif s.type == "wkv":
                 # previous token's input row + one matrix per head
                 total += self.hidden_size + s.mixer["heads"] * s.mixer["dim"] ** 2
+            elif s.type == "retention":
+                total += s.mixer["heads"] * s.mixer["dim"] * s.mixer["vdim"]
+            elif s.type == "mlstm":
+                # matrix, normaliser vector and running maximum per head
+                total += s.mixer["heads"] * (s.mixer["dim"] * (s.mixer["vdim"] + 1) + 1)
             elif s.type == "parallel":
                 right = s.mixer["right"]
                 total += right["heads"] * right["dim"] * right["vdim"]

@@ -21,6 +21,11 @@ arguments, so another model family can assemble them differently.
   * `MatrixStateMixer`, `GeluMLP` — matrix-state recurrences.
   * `GatedReluMLP`, `GroupRoutedExpertsMLP` — gated feed-forward and routed
     experts with a softmax router, group-limited choice and identity experts.
+  * `ScalarDecayMixer` — matrix-state recurrences whose decay is one number
+    per head: fixed (retention) or gated per token (mLSTM).
+  * `ReluSquaredExpertsMLP` — routed squared-ReLU experts beside a shared one.
+  * `TokenTableGate` — a per-layer token table that enters the residual
+    through a gate and a norm.
 
 Projections are library GEMMs over fused weights (one GEMM in, one out per
 block); everything between them is one HIP kernel each (ops layer).
@@ -239,33 +244,51 @@ class LatentAttention(nn.Module):
 
     which is exact because a softmax with a sink is still linear in the
     values.  Optional per-head sink in the softmax denominator, optional
-    sigmoid output gate on the concatenated heads.  Rotation is interleaved
-    pairs over the first `rot_dims` entries of the rotated part.
+    sigmoid output gate: one entry per output element (out_gate) or one
+    number per head (head_gate, applied to o_lat inside the attention
+    kernel, which commutes with W_uv).  Rotation is interleaved pairs over
+    the first `rot_dims` entries of the rotated part.
+
+    q_rank 0: queries are projected directly, without a normed query latent.
+    own_rows False: the layer caches nothing and has no down-projection; the
+    cache handed to it holds another layer's rows.
+
+    The block can be used whole (`forward`) or between GEMMs that a model
+    fuses with others (`mix`: from the input projection to the gated heads).
     """
 
     def __init__(
         self, hidden: int, heads: int, dim: int, rot_dim: int, vdim: int, q_rank: int,
         kv_rank: int, scale: float, rot_base: float, rot_dims: int, eps: float,
-        sink: bool = True, out_gate: bool = True, device="cpu", dtype=torch.bfloat16,
+        sink: bool = True, out_gate: bool = True, head_gate: bool = False,
+        own_rows: bool = True, device="cpu", dtype=torch.bfloat16,
     ) -> None:
         super().__init__()
         assert 0 <= rot_dims <= rot_dim and rot_dims % 2 == 0
+        assert not (out_gate and head_gate)
         self.heads, self.dim, self.rot_dim, self.vdim = heads, dim, rot_dim, vdim
         self.q_rank, self.kv_rank = q_rank, kv_rank
         self.scale, self.eps = float(scale), float(eps)
-        self.out_gate = out_gate
+        self.out_gate, self.head_gate, self.own_rows = out_gate, head_gate, own_rows
         self.row = kv_rank + rot_dim  # one cache row
+        self.n_out = heads * vdim
         s = 1.0 / math.sqrt(hidden)
-        self.n_in = q_rank + kv_rank + rot_dim
-        self.ng = heads * vdim if out_gate else 0
-        # rows: query latent | key/value latent | shared rotated key part | gate
+        self.nq = q_rank if q_rank > 0 else heads * (dim + rot_dim)
+        self.n_in = self.nq + (self.row if own_rows else 0)
+        self.ng = heads * vdim if out_gate else (heads if head_gate else 0)
+        # rows: query latent (or queries) | key/value latent | shared rotated
+        # key part | gate
         self.w_in = _param((self.n_in + self.ng, hidden), device, dtype, s)
-        self.q_norm = _param((q_rank,), device, dtype, None)
-        self.kv_norm = _param((kv_rank,), device, dtype, None)
+        self.kv_norm = _param((kv_rank,), device, dtype, None) if own_rows else None
+        self.q_norm = self.w_uq = None
         with torch.no_grad():
-            self.q_norm.fill_(1.0)
-            self.kv_norm.fill_(1.0)
-        self.w_uq = _param((heads * (dim + rot_dim), q_rank), device, dtype, 1.0 / math.sqrt(q_rank))
+            if own_rows:
+                self.kv_norm.fill_(1.0)
+        if q_rank > 0:
+            self.q_norm = _param((q_rank,), device, dtype, None)
+            with torch.no_grad():
+                self.q_norm.fill_(1.0)
+            self.w_uq = _param((heads * (dim + rot_dim), q_rank), device, dtype, 1.0 / math.sqrt(q_rank))
         # per head, laid out for batched GEMMs: [H, dim, kv_rank] and [H, kv_rank, vdim]
         self.w_uk = _param((heads, dim, kv_rank), device, dtype, 1.0 / math.sqrt(kv_rank))
         self.w_uv = _param((heads, kv_rank, vdim), device, dtype, 1.0 / math.sqrt(kv_rank))
@@ -278,19 +301,23 @@ class LatentAttention(nn.Module):
             "inv_freq", ops.rotary_inv_freq(rot_base, rot_dims, device), persistent=False
         )
 
-    def cache_spec(self) -> dict:
-        return {"kind": "latent", "row": self.row}
+    def cache_spec(self):
+        return {"kind": "latent", "row": self.row} if self.own_rows else []
 
     def load(self, get, prefix: str) -> None:
         H, D, R = self.heads, self.dim, self.kv_rank
-        parts = [get(prefix + "dq"), get(prefix + "dkv")]
-        if self.out_gate:
+        parts = [get(prefix + ("dq" if self.q_rank > 0 else "q"))]
+        if self.own_rows:
+            parts.append(get(prefix + "dkv"))
+        if self.ng:
             parts.append(get(prefix + "g"))
         with torch.no_grad():
             self.w_in.copy_(torch.cat(parts, dim=0))
-            self.q_norm.copy_(get(prefix + "dq.norm"))
-            self.kv_norm.copy_(get(prefix + "dkv.norm"))
-            self.w_uq.copy_(get(prefix + "uq"))
+            if self.own_rows:
+                self.kv_norm.copy_(get(prefix + "dkv.norm"))
+            if self.q_rank > 0:
+                self.q_norm.copy_(get(prefix + "dq.norm"))
+                self.w_uq.copy_(get(prefix + "uq"))
             self.w_uk.copy_(get(prefix + "uk").view(H, D, R))
             self.w_uv.copy_(get(prefix + "uv").view(H, self.vdim, R).transpose(1, 2))
             if self.sink is not None:
@@ -300,21 +327,35 @@ class LatentAttention(nn.Module):
     def mfma_rows(self, dtype, on_gpu: bool) -> bool:
         return ops.latent_rows_supported(dtype, self.row, self.kv_rank, on_gpu)
 
-
     def forward(self, h, positions, cache, meta):
+        return _mm(self.mix(_mm(h, self.w_in), positions, cache, meta), self.w_o)
+
+    def mix(self, proj, positions, cache, meta, out: Optional[torch.Tensor] = None):
+        """proj [rows, >= n_in + gate columns], the fused input projection;
+        returns the gated heads [rows, n_out], written to `out` (may be a
+        column block of wider rows) when given."""
         lat_cache = cache[0]
         H, D, Rr, Rk = self.heads, self.dim, self.rot_dim, self.kv_rank
-        rows = h.shape[0]
-        proj = _mm(h, self.w_in)
-        cq = ops.latent_kv_prep(
-            proj, self.q_rank, Rk, Rr, self.q_norm, self.kv_norm, self.eps, self.inv_freq,
-            positions, meta.slot_mapping, lat_cache,
-        )
-        q = _mm(cq, self.w_uq)  # [rows, H*(D+Rr)]
+        rows = proj.shape[0]
+        if self.q_rank > 0:
+            q = ops.latent_kv_prep(
+                proj, self.q_rank, Rk, Rr, self.q_norm, self.kv_norm, self.eps, self.inv_freq,
+                positions, meta.slot_mapping, lat_cache,
+            )
+            q = _mm(q, self.w_uq)  # [rows, H*(D+Rr)]
+        else:
+            q = proj[:, : self.nq]
+            if self.own_rows:
+                ops.latent_kv_prep(
+                    proj[:, self.nq :], 0, Rk, Rr, None, self.kv_norm, self.eps, self.inv_freq,
+                    positions, meta.slot_mapping, lat_cache,
+                )
+        gate = proj[:, self.n_in : self.n_in + self.ng] if self.ng else None
+        head_gate = gate if self.head_gate else None
         qa = torch.empty(rows, H, self.row, dtype=q.dtype, device=q.device)
         # latent-space query part: per head q_un @ W_uk, written in place
         torch.bmm(
-            q.view(rows, H, D + Rr)[:, :, :D].transpose(0, 1), self.w_uk,
+            q.unflatten(1, (H, D + Rr))[:, :, :D].transpose(0, 1), self.w_uk,
             out=qa[:, :, :Rk].transpose(0, 1),
         )
         ops.rotate_pack_queries(q, H, D, Rr, self.inv_freq, positions, qa, Rk)
@@ -331,19 +372,23 @@ class LatentAttention(nn.Module):
             ops.latent_attention_rows(
                 qa, lat_cache, Rk, meta.seq_block_tables, meta.seg_start, meta.seg_len,
                 meta.seg_ctx, meta.max_seg_len, self.scale, H, sink=self.sink, out=o,
+                gate=head_gate,
             )
         else:
             o = ops.paged_attention_general(
                 qa, lat_cache, v_view, meta.seq_block_tables, meta.tok_seq, positions,
-                self.scale, H, sink=self.sink,
+                self.scale, H, sink=self.sink, gate=head_gate, gate_per_head=self.head_gate,
             )
         # values: per head o_lat @ W_uv, heads concatenated in place
-        ov = torch.empty(rows, H, self.vdim, dtype=q.dtype, device=q.device)
-        torch.bmm(o.view(rows, H, Rk).transpose(0, 1), self.w_uv, out=ov.transpose(0, 1))
-        ov = ov.view(rows, H * self.vdim)
+        if out is None:
+            out = torch.empty(rows, self.n_out, dtype=q.dtype, device=q.device)
+        torch.bmm(
+            o.view(rows, H, Rk).transpose(0, 1), self.w_uv,
+            out=out.unflatten(1, (H, self.vdim)).transpose(0, 1),
+        )
         if self.out_gate:
-            ops.sigmoid_gate_mul(ov, proj[:, self.n_in :])
-        return _mm(ov, self.w_o)
+            ops.sigmoid_gate_mul(out, gate)
+        return out
 
 
 class ReluSquaredMLP(nn.Module):
@@ -778,6 +823,111 @@ class MatrixStateMixer(nn.Module):
         return F.linear(g, self.w_o)
 
 
+class ScalarDecayMixer(nn.Module):
+    """Matrix-state recurrences whose state decays by ONE number per head and
+    token, scanned by `ops.matrix_state_scan`; per-head outputs divided by
+    their root mean square, gated, heads concatenated.
+
+    kind "retention": fixed decay per head, rotate-half positions on q and k
+    (the first rot_dims entries), k scaled by dim^-1/2, silu gate.
+
+    kind "mlstm": input and forget gates per head and token (log gates capped
+    by gate_cap), a normaliser vector and a running maximum beside the
+    matrix; q scaled by dim^-1/2; a weight on the normed heads, sigmoid gate.
+    The gates' logits are computed in fp32 by whoever runs the layer's small
+    projections: `w_small` holds their rows, [i | f].
+
+    Rows of w_in: q | k | v | gate.  `mix` goes from the projections to the
+    gated heads, so that a model can fuse both GEMMs with others.
+    """
+
+    def __init__(
+        self, hidden: int, kind: str, heads: int, dim: int, vdim: int, eps: float,
+        decay=None, rot_base: float = 10000.0, rot_dims: int = 0, gate_cap: float = 1.0,
+        device="cpu", dtype=torch.bfloat16,
+    ) -> None:
+        super().__init__()
+        assert kind in ("retention", "mlstm") and 0 <= rot_dims <= dim and rot_dims % 2 == 0
+        self.kind, self.heads, self.dim, self.vdim, self.eps = kind, heads, dim, vdim, float(eps)
+        self.nk, self.nv = heads * dim, heads * vdim
+        self.n_out = self.nv
+        self.gate_cap = float(gate_cap)
+        self.w_in = _param((2 * self.nk + 2 * self.nv, hidden), device, dtype, 1.0 / math.sqrt(hidden))
+        self.w_o = _param((hidden, self.nv), device, dtype, 1.0 / math.sqrt(self.nv))
+        self.norm = self.w_small = self.head_decay = None
+        f32 = dict(device=device, dtype=torch.float32)
+        if kind == "retention":
+            self.head_decay = nn.Parameter(
+                torch.tensor([float(d) for d in decay], **f32), requires_grad=False
+            )
+            assert self.head_decay.shape == (heads,)
+        else:
+            self.norm = _param((self.nv,), device, dtype, None)
+            with torch.no_grad():
+                self.norm.fill_(1.0)
+            self.w_small = _param((2 * heads, hidden), device, dtype, 1.0 / math.sqrt(hidden))
+            # the gates' biases enter the recurrence: fp32
+            self.b_i = nn.Parameter(torch.full((heads,), -3.0, **f32), requires_grad=False)
+            self.b_f = nn.Parameter(torch.full((heads,), 4.0, **f32), requires_grad=False)
+        self.rot_key = (float(rot_base), int(rot_dims))
+        self.register_buffer(
+            "inv_freq",
+            ops.rotary_inv_freq(rot_base, rot_dims, device) if rot_dims > 0 else None,
+            persistent=False,
+        )
+
+    def cache_spec(self) -> dict:
+        width = ops.matrix_state_width(self.heads, self.dim, self.vdim, self.kind == "mlstm")
+        return {"kind": "state", "width": width}
+
+    def load(self, get, prefix: str) -> None:
+        with torch.no_grad():
+            self.w_in.copy_(torch.cat([get(prefix + n) for n in "qkvg"], dim=0))
+            self.w_o.copy_(get(prefix + "o"))
+            if self.kind == "mlstm":
+                self.norm.copy_(get(prefix + "norm"))
+                self.w_small.copy_(torch.cat([get(prefix + "i"), get(prefix + "f")], dim=0))
+                self.b_i.copy_(get(prefix + "i.b").float())
+                self.b_f.copy_(get(prefix + "f.b").float())
+
+    def forward(self, h, positions, cache, meta):
+        small = ops.small_projection(h, self.w_small) if self.w_small is not None else None
+        return _mm(self.mix(_mm(h, self.w_in), small, positions, cache, meta), self.w_o)
+
+    def mix(
+        self, proj, small, positions, cache, meta, out: Optional[torch.Tensor] = None,
+        tables: Optional[dict] = None,
+    ):
+        """proj [rows, >= q | k | v | gate], small fp32 [rows, i | f] (mlstm);
+        `tables` keeps rotation tables between the layers of one step."""
+        (state,) = cache
+        a, b, c = self.nk, 2 * self.nk, 2 * self.nk + self.nv
+        q, k, v, gate = proj[:, :a], proj[:, a:b], proj[:, b:c], proj[:, c : c + self.nv]
+        seg = (meta.seg_start, meta.seg_len, meta.seg_slot, meta.seg_fresh)
+        sizes = (self.heads, self.dim, self.vdim)
+        if self.kind == "retention":
+            rot = None
+            if self.inv_freq is not None:
+                tables = {} if tables is None else tables
+                if self.rot_key not in tables:
+                    tables[self.rot_key] = ops.rotary_table(positions, self.inv_freq)
+                rot = tables[self.rot_key]
+            o = ops.matrix_state_scan(
+                q, k, v, state, *seg, *sizes, head_decay=self.head_decay, rot=rot,
+                k_scale=self.dim ** -0.5,
+            )
+        else:
+            o = ops.matrix_state_scan(
+                q, k, v, state, *seg, *sizes, gates=(small[:, : self.heads], small[:, self.heads :]),
+                gate_bias=(self.b_i, self.b_f), gate_cap=self.gate_cap, q_scale=self.dim ** -0.5,
+            )
+        MatrixStateMixer._zero_pad_rows(o, meta)
+        return ops.group_rms_norm_gate(
+            o, gate, self.norm, self.vdim, "silu" if self.kind == "retention" else "sigmoid",
+            self.eps, out=out,
+        )
+
+
 class GeluMLP(nn.Module):
     """down(gelu(up h)) with the exact (erf) gelu."""
 
@@ -915,3 +1065,96 @@ class GroupRoutedExpertsMLP(nn.Module):
         xe = ops.scale_gather_rows(h, gather, (gather >= 0).float())
         ye = self._experts(xe.view(E, cap, hidden), cap)
         return ops.routed_combine(ye, h, rows.contiguous(), w)
+
+
+class ReluSquaredExpertsMLP(nn.Module):
+    """Routed experts down(relu(up h)^2) whose weights are the softmax over
+    the chosen router logits, optionally beside a shared expert of the same
+    form that runs for every token.
+
+    The router's rows (`w_small`) are computed in fp32, by `route` or by a
+    model that shares the product with other small projections.  `experts_of`
+    returns the experts' outputs with the rows and weights of every token's
+    choices, so that a model can join the weighted sum to its residual.
+
+    Dispatch as `GroupRoutedExpertsMLP`.
+    """
+
+    def __init__(
+        self, hidden: int, ff: int, experts: int, top: int, shared_ff: int = 0,
+        device="cpu", dtype=torch.bfloat16,
+    ) -> None:
+        super().__init__()
+        assert 1 <= top <= experts
+        self.experts, self.top, self.ff = experts, top, ff
+        s = 1.0 / math.sqrt(hidden)
+        self.w_small = _param((experts, hidden), device, dtype, s)
+        # pre-transposed for bmm: [E, hidden, ff] and [E, ff, hidden]
+        self.w1 = _param((experts, hidden, ff), device, dtype, s)
+        self.w2 = _param((experts, ff, hidden), device, dtype, 1.0 / math.sqrt(ff))
+        self.shared = (
+            ReluSquaredMLP(hidden, shared_ff, device=device, dtype=dtype) if shared_ff > 0 else None
+        )
+
+    def load(self, get, prefix: str) -> None:
+        with torch.no_grad():
+            self.w_small.copy_(get(prefix + "router"))
+            for e in range(self.experts):
+                self.w1[e].copy_(get(f"{prefix}e{e}.up").t())
+                self.w2[e].copy_(get(f"{prefix}e{e}.down").t())
+        if self.shared is not None:
+            self.shared.load(get, prefix + "shared.")
+
+    def route(self, z: torch.Tensor):
+        """fp32 logits [T, experts] (may be a column block) -> idx int32, weights fp32."""
+        return ops.grouped_topk_route(z, None, self.top)
+
+    def _experts(self, xe: torch.Tensor, rows: int) -> torch.Tensor:
+        """xe [E, rows, hidden] -> [E * rows, hidden]."""
+        E = self.experts
+        act = ops.relu_squared(torch.bmm(xe, self.w1).view(E * rows, self.ff))
+        return torch.bmm(act.view(E, rows, self.ff), self.w2).view(E * rows, -1)
+
+    def experts_of(self, h, z, meta=None) -> dict:
+        """Arguments of `ops.residual_routed_add`: ye, w and rows or idx."""
+        T, hidden = h.shape
+        E = self.experts
+        idx, w = self.route(z)
+        if meta is not None and meta.num_prefill_tokens == 0:
+            ye = self._experts(h.unsqueeze(0).expand(E, T, hidden), T)
+            return dict(ye=ye, w=w, idx=idx, experts=E)
+        gather, rows, cap = expert_dispatch_plan(idx.long(), E)
+        xe = ops.scale_gather_rows(h, gather, (gather >= 0).float())
+        return dict(ye=self._experts(xe.view(E, cap, hidden), cap), w=w, rows=rows.contiguous())
+
+    def forward(self, h, meta=None):
+        c = self.experts_of(h, ops.small_projection(h, self.w_small), meta)
+        y = ops.routed_combine(
+            c["ye"], h, c.get("rows"), c["w"], idx=c.get("idx"), experts=c.get("experts", 0)
+        )
+        return y if self.shared is None else y + self.shared(h)
+
+
+class TokenTableGate(nn.Module):
+    """What a per-layer token table adds to the residual: the table's row e of
+    the token (dim entries per layer), gated by the residual and projected
+    back, y = W_proj (gelu_tanh(W_gate x) * e); `norm` is the weight of the
+    RMS norm that y passes on its way into the residual."""
+
+    def __init__(self, hidden: int, dim: int, device="cpu", dtype=torch.bfloat16) -> None:
+        super().__init__()
+        self.w_gate = _param((dim, hidden), device, dtype, 1.0 / math.sqrt(hidden))
+        self.w_proj = _param((hidden, dim), device, dtype, 1.0 / math.sqrt(dim))
+        self.norm = _param((hidden,), device, dtype, None)
+        with torch.no_grad():
+            self.norm.fill_(1.0)
+
+    def load(self, get, prefix: str) -> None:
+        with torch.no_grad():
+            self.w_gate.copy_(get(prefix + "gate"))
+            self.w_proj.copy_(get(prefix + "proj"))
+            self.norm.copy_(get(prefix + "norm"))
+
+    def forward(self, x, table, tokens):
+        """x: the residual in the activation dtype; table: this layer's columns."""
+        return _mm(ops.gelu_tanh_table_mul(_mm(x, self.w_gate), table, tokens), self.w_proj)

@@ -80,7 +80,20 @@ def _vemenex_config(raw: dict, path: str) -> ModelConfig:
     return config_from_json(raw, path)
 
 
+def _garesun_factory(cfg, device, dtype, tp):
+    from .garesun import GaresunForCausalLM
+
+    return GaresunForCausalLM(cfg, device=device, dtype=dtype, tp=tp)
+
+
+def _garesun_config(raw: dict, path: str) -> ModelConfig:
+    from .garesun import config_from_json
+
+    return config_from_json(raw, path)
+
+
 register_architecture("llama", None, _llama_factory)
+register_architecture("garesun", _garesun_config, _garesun_factory)
 register_architecture("vemenex", _vemenex_config, _vemenex_factory)
 register_architecture("potatar", _potatar_config, _potatar_factory)
 register_architecture("lopovik", _lopovik_config, _lopovik_factory)

@@ -674,6 +674,7 @@ def latent_attention_rows(
     q, cache, v_dim: int, block_tables, seg_start, seg_len, seg_ctx, max_seg_len: int,
     scale: float, num_heads: int, sink: Optional[torch.Tensor] = None,
     out: Optional[torch.Tensor] = None, nsplit: int = 0,
+    gate: Optional[torch.Tensor] = None,
 ) -> torch.Tensor:
     """Causal multi-query attention of every segment of the step (prompt
     portions and single tokens alike) over the paged latent cache
@@ -693,6 +694,8 @@ def latent_attention_rows(
         assert t.dtype == torch.int32 and t.is_contiguous()
     S = seg_start.shape[0]
     assert block_tables.shape[0] >= S and seg_len.shape[0] == S and seg_ctx.shape[0] == S
+    if gate is not None:
+        assert gate.shape == (R, num_heads) and gate.stride(1) == 1 and gate.dtype == q.dtype
     if sink is not None:
         assert sink.dtype == torch.float32 and sink.shape == (num_heads,) and sink.is_contiguous()
     if out is None:
@@ -704,7 +707,8 @@ def latent_attention_rows(
     if nsplit > 1:
         scratch = split_scratch(q.device, R * num_heads * nsplit * (v_dim + 4))
     rc = _hl().lig_latent_attention_rows(
-        _ptr(out), _ptr(q), _ptr(cache), _ptr(sink), _ptr(seg_start), _ptr(seg_len),
+        _ptr(out), _ptr(q), _ptr(cache), _ptr(sink), _ptr(gate),
+        0 if gate is None else gate.stride(0), _ptr(seg_start), _ptr(seg_len),
         _ptr(seg_ctx), _ptr(block_tables), block_tables.shape[1], float(scale), S,
         int(max_seg_len), num_heads, row, v_dim, bs, int(nsplit), _ptr(scratch), _stream(),
     )
@@ -790,7 +794,8 @@ def latent_kv_prep(
     """Per row of the fused projection [query latent | key/value latent |
     shared rotated key part | ...]: returns the RMS-normed query latent and
     writes [normed key/value latent | rotated key part] into the paged latent
-    cache [blocks, 1, block_size, kv_rank + rot_dim] at slot_mapping."""
+    cache [blocks, 1, block_size, kv_rank + rot_dim] at slot_mapping.
+    q_rank 0 (w_q None): the rows hold no query latent."""
     if _use_hybrid(proj):
         R = proj.shape[0]
         assert proj.stride(1) == 1 and proj.shape[1] >= q_rank + kv_rank + rot_dim
@@ -812,26 +817,66 @@ def latent_kv_prep(
 
 def rotate_pack_queries(q, heads: int, dim: int, rot_dim: int, inv_freq, positions, out, lead: int):
     """out[r, h, lead:] = interleaved rotation of q[r, h, dim:dim+rot_dim];
-    q [R, heads*(dim+rot_dim)] contiguous, out [R, heads, lead+rot_dim]."""
+    q [R, heads*(dim+rot_dim)] (may be a column block of wider rows), out
+    [R, heads, lead+rot_dim]."""
     if _use_hybrid(q):
         R = q.shape[0]
-        assert q.is_contiguous() and out.is_contiguous() and out.dtype == q.dtype
+        assert q.stride(1) == 1 and q.shape[1] == heads * (dim + rot_dim)
+        assert out.is_contiguous() and out.dtype == q.dtype
         assert out.shape == (R, heads, lead + rot_dim) and positions.dtype == torch.int64
         _hl().lig_rotate_pack_queries(
-            _ptr(out), _ptr(q), _ptr(inv_freq), inv_freq.shape[0], _ptr(positions), R,
+            _ptr(out), _ptr(q), q.stride(0), _ptr(inv_freq), inv_freq.shape[0], _ptr(positions), R,
             heads, dim, rot_dim, lead, _is_f32(q), _stream(),
         )
         return out
     return torch_ref.rotate_pack_queries(q, heads, dim, rot_dim, inv_freq, positions, out, lead)
 
 
-def relu_squared(x: torch.Tensor) -> torch.Tensor:
+def rotary_table(positions: torch.Tensor, inv_freq: torch.Tensor) -> torch.Tensor:
+    """fp32 [R, 2n]: cosines, then sines, of positions[r] * inv_freq[i]; one
+    table serves every layer of a step that rotates the same way."""
+    if _use_hybrid(positions):
+        assert positions.dtype == torch.int64 and inv_freq.dtype == torch.float32
+        R, n = positions.shape[0], inv_freq.shape[0]
+        cs = torch.empty(R, 2 * n, dtype=torch.float32, device=positions.device)
+        _hl().lig_rotary_table(_ptr(cs), _ptr(positions), _ptr(inv_freq), R, n, _stream())
+        return cs
+    return torch_ref.rotary_table(positions, inv_freq)
+
+
+def relu_squared(x: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """relu(x)^2; with `out` (2-D), x and out may be column blocks of wider rows."""
+    if out is not None:
+        assert x.dim() == 2 and out.shape == x.shape and out.dtype == x.dtype
+        assert x.stride(1) == 1 and out.stride(1) == 1
+        if _use_hybrid(x):
+            _hl().lig_relu_squared_rows(
+                _ptr(out), out.stride(0), _ptr(x), x.stride(0), x.shape[0], x.shape[1],
+                _is_f32(x), _stream(),
+            )
+            return out
+        return out.copy_(torch_ref.relu_squared(x))
     if _use_hybrid(x):
         assert x.is_contiguous()
         out = torch.empty_like(x)
         _hl().lig_relu_squared(_ptr(out), _ptr(x), x.numel(), _is_f32(x), _stream())
         return out
     return torch_ref.relu_squared(x)
+
+
+def gelu_tanh_table_mul(z: torch.Tensor, table: torch.Tensor, tokens: torch.Tensor) -> torch.Tensor:
+    """out[r] = gelu_tanh(z[r]) * table[tokens[r]] (the tanh form of gelu);
+    z [R, F] contiguous, table [vocab, F] may be a column block."""
+    assert z.dim() == 2 and table.shape[1] == z.shape[1] and table.dtype == z.dtype
+    if _use_hybrid(z):
+        assert z.is_contiguous() and table.stride(1) == 1 and tokens.dtype == torch.int64
+        out = torch.empty_like(z)
+        _hl().lig_gelu_tanh_table_mul(
+            _ptr(out), _ptr(z), _ptr(table), table.stride(0), _ptr(tokens), z.shape[0],
+            z.shape[1], _is_f32(z), _stream(),
+        )
+        return out
+    return torch_ref.gelu_tanh_table_mul(z, table, tokens)
 
 
 def silu_mul(x: torch.Tensor) -> torch.Tensor:
@@ -1100,23 +1145,34 @@ def token_shift_mix(x, mu, state, tok_seq, seg_start, seg_len, seg_slot, seg_fre
 MATRIX_STATE_KEY_CLASSES = (4, 8, 12, 16, 24, 32, 48, 64)
 
 
-def matrix_state_width(heads: int, dim: int, vdim: int) -> int:
-    """fp32 entries of one sequence's matrix state: the scan kernel splits a
-    head's key channels over 8 lanes (heads of 32 or more key channels whose
-    8 * vdim threads fit a workgroup) or 4, and keeps the state in the order
-    its threads hold it, key channels padded to the split times the kernel's
-    size class."""
-    split = 8 if dim >= 32 and vdim * 8 <= 1024 else 4
+# value columns per workgroup of the scan kernel
+MATRIX_STATE_COLUMNS = 64
+
+
+def matrix_state_width(heads: int, dim: int, vdim: int, gated: bool = False) -> int:
+    """fp32 entries of one sequence's matrix state: the scan kernel walks
+    blocks of up to 64 value columns, splits a head's key channels over 8
+    lanes (heads of 32 or more key channels) or 4, and keeps the state in the
+    order its threads hold it, key channels padded to the split times the
+    kernel's size class and value columns to whole blocks.  The gated form
+    adds the normaliser column and the running maximum of every block."""
+    split = 8 if dim >= 32 else 4
     need = (dim + split - 1) // split
     kpt = next((c for c in MATRIX_STATE_KEY_CLASSES if c >= need), None)
     if kpt is None:
-        raise ValueError(f"matrix-state heads hold at most 256 key channels, got {dim}")
-    return heads * split * kpt * vdim
+        raise ValueError(f"matrix-state heads hold at most 512 key channels, got {dim}")
+    cols = min(vdim, MATRIX_STATE_COLUMNS)
+    blocks = (vdim + cols - 1) // cols
+    if gated:
+        return heads * blocks * (split * kpt * (cols + 1) + 1)
+    return heads * blocks * split * kpt * cols
 
 
 def matrix_state_scan(
     q, k, v, state, seg_start, seg_len, seg_slot, seg_fresh, heads: int, dim: int,
     vdim: int, decay_pre=None, head_decay=None, bonus=None, act_silu: bool = False,
+    gates=None, gate_bias=None, gate_cap: float = 1.0, rot: Optional[torch.Tensor] = None,
+    q_scale: float = 1.0, k_scale: float = 1.0,
 ) -> torch.Tensor:
     """Linear recurrences with one [dim, vdim] fp32 state matrix S per head,
     over the segments of the flat batch; q, k [R, heads*dim] and v
@@ -1127,18 +1183,43 @@ def matrix_state_scan(
         w_t = exp(-exp(decay_pre_t))
     With head_decay d (fp32 [heads]):
         S <- d_h S + k_t v_t^T;  o_t = S^T q_t
-    act_silu applies silu to q, k, v on the way in.  state [slots,
+    With gates = (i, f) (fp32 [R, heads] each, one row stride; may be column
+    blocks) and gate_bias = (b_i, b_f) (fp32 [heads]): log gates
+        i_t = cap tanh((i + b_i) / cap),  f_t = logsigmoid(cap tanh((f + b_f) / cap)),
+        m_t = max(f_t + m_{t-1}, i_t),  m = 0 at the start,
+        S <- exp(f_t + m_{t-1} - m_t) S + exp(i_t - m_t) k_t v_t^T;  n likewise with k_t,
+        o_t = S^T q_t / (max(|n . q_t|, exp(-m_t)) + 1e-6)
+    On the way in, in this order: act_silu applies silu to q, k, v; `rot`
+    (fp32 [R, 2n] from rotary_table) turns entries i and i + n of every q and
+    k head; q_scale and k_scale multiply.  state [slots,
     matrix_state_width] is read unless the segment starts its sequence and
     written back; its layout is private to the implementation.  Returns fp32
     [R, heads*vdim]; rows of no segment are left untouched (undefined)."""
-    assert (bonus is None) == (decay_pre is None) and (bonus is None) != (head_decay is None)
+    assert (bonus is None) == (decay_pre is None)
+    assert sum(t is not None for t in (bonus, head_decay, gates)) == 1
+    assert (gates is None) == (gate_bias is None)
     assert state.dtype == torch.float32
     if _use_hybrid(q):
         R = q.shape[0]
         assert q.shape[1] == heads * dim and k.shape[1] == heads * dim and v.shape[1] == heads * vdim
         assert q.stride(1) == 1 and k.stride(1) == 1 and v.stride(1) == 1
         assert q.dtype == k.dtype == v.dtype
-        assert state.is_contiguous() and state.shape[1] == matrix_state_width(heads, dim, vdim)
+        assert state.is_contiguous() and state.shape[1] == matrix_state_width(
+            heads, dim, vdim, gates is not None
+        )
+        gi = gf = bi = bf = None
+        if gates is not None:
+            (gi, gf), (bi, bf) = gates, gate_bias
+            for g in gates:
+                assert g.dtype == torch.float32 and g.shape == (R, heads) and g.stride(1) == 1
+                assert g.stride(0) == gi.stride(0)
+            for b in gate_bias:
+                assert b.dtype == torch.float32 and b.shape == (heads,) and b.is_contiguous()
+        nf = 0
+        if rot is not None:
+            nf = rot.shape[1] // 2
+            assert rot.dtype == torch.float32 and rot.is_contiguous() and rot.shape == (R, 2 * nf)
+            assert 2 * nf <= dim
         for t, n in ((decay_pre, R * heads * dim), (bonus, heads * dim), (head_decay, heads)):
             if t is not None:
                 assert t.dtype == torch.float32 and t.is_contiguous() and t.numel() == n
@@ -1146,36 +1227,44 @@ def matrix_state_scan(
         out = torch.empty(R, heads * vdim, dtype=torch.float32, device=q.device)
         rc = _hl().lig_matrix_state_scan(
             _ptr(out), _ptr(q), q.stride(0), _ptr(k), k.stride(0), _ptr(v), v.stride(0),
-            _ptr(decay_pre), _ptr(head_decay), _ptr(bonus), _ptr(state), state.stride(0),
+            _ptr(decay_pre), _ptr(head_decay), _ptr(bonus), _ptr(gi), _ptr(gf),
+            0 if gi is None else gi.stride(0), _ptr(bi), _ptr(bf), float(gate_cap), _ptr(rot), nf,
+            float(q_scale), float(k_scale), _ptr(state), state.stride(0),
             _ptr(seg_start), _ptr(seg_len), _ptr(seg_slot), _ptr(seg_fresh), S, heads, dim,
             vdim, int(bool(act_silu)), _is_f32(q), _stream(),
         )
         if rc != 0:
-            raise RuntimeError("matrix_state_scan: keys or values wider than 256 per head")
+            raise RuntimeError("matrix_state_scan: more than 512 key channels per head")
         return out
     return torch_ref.matrix_state_scan(
         q, k, v, state, seg_start, seg_len, seg_slot, seg_fresh, heads, dim, vdim,
-        decay_pre, head_decay, bonus, act_silu,
+        decay_pre, head_decay, bonus, act_silu, gates, gate_bias, gate_cap, rot, q_scale, k_scale,
     )
 
 
-def group_rms_norm_gate(o, gate, w, group: int, gate_act: str, eps: float) -> torch.Tensor:
+def group_rms_norm_gate(
+    o, gate, w, group: int, gate_act: str, eps: float, out: Optional[torch.Tensor] = None
+) -> torch.Tensor:
     """o fp32 [R, C]: every `group` consecutive entries are divided by their
-    root mean square (group == C: the whole row), then times w [C], times
-    silu(gate) or sigmoid(gate); gate [R, C] may be a column-block view.
-    Result in w's dtype."""
+    root mean square (group == C: the whole row), then times w [C] (None: no
+    weight), times silu(gate) or sigmoid(gate); gate [R, C] may be a
+    column-block view.  Result in the gate's dtype; `out` may be a column
+    block of wider rows."""
     assert o.dtype == torch.float32 and gate_act in ("silu", "sigmoid")
     R, C = o.shape
-    assert C % group == 0 and gate.shape == (R, C) and w.shape == (C,)
+    assert C % group == 0 and gate.shape == (R, C)
+    assert w is None or (w.shape == (C,) and w.dtype == gate.dtype)
+    if out is None:
+        out = torch.empty(R, C, dtype=gate.dtype, device=o.device)
+    assert out.shape == (R, C) and out.dtype == gate.dtype and out.stride(1) == 1
     if _use_hybrid(o):
-        assert o.is_contiguous() and gate.stride(1) == 1 and gate.dtype == w.dtype
-        out = torch.empty(R, C, dtype=w.dtype, device=o.device)
+        assert o.is_contiguous() and gate.stride(1) == 1
         _hl().lig_group_rms_norm_gate(
-            _ptr(out), _ptr(o), _ptr(gate), gate.stride(0), _ptr(w), int(group),
-            1 if gate_act == "silu" else 0, float(eps), R, C, _is_f32(w), _stream(),
+            _ptr(out), out.stride(0), _ptr(o), _ptr(gate), gate.stride(0), _ptr(w), int(group),
+            1 if gate_act == "silu" else 0, float(eps), R, C, _is_f32(gate), _stream(),
         )
         return out
-    return torch_ref.group_rms_norm_gate(o, gate, w, group, gate_act, eps, w.dtype)
+    return out.copy_(torch_ref.group_rms_norm_gate(o, gate, w, group, gate_act, eps, gate.dtype))
 
 
 def gelu_erf(x: torch.Tensor) -> torch.Tensor:
@@ -1252,8 +1341,9 @@ def grouped_topk_route(
     `keep` groups (of N/groups neighbours) with the largest best choice score
     can be chosen; the `top` largest choice scores win (ties: lower index).
     Returns (idx int32 [T, top], weights fp32 [T, top] = chosen s over their
-    sum + 1e-20)."""
-    assert z.dtype == torch.float32 and z.dim() == 2 and z.is_contiguous()
+    sum + 1e-20).  z may be a column block of wider rows.  With one group and
+    no correction the weights are the softmax over the chosen logits."""
+    assert z.dtype == torch.float32 and z.dim() == 2 and z.stride(1) == 1
     T, N = z.shape
     assert N % groups == 0 and 1 <= keep <= groups and 1 <= top <= keep * (N // groups)
     if correction is not None:
@@ -1262,7 +1352,7 @@ def grouped_topk_route(
         idx = torch.empty(T, top, dtype=torch.int32, device=z.device)
         w = torch.empty(T, top, dtype=torch.float32, device=z.device)
         rc = _hl().lig_grouped_topk_route(
-            _ptr(z), _ptr(correction), T, N, groups, keep, top, _ptr(idx), _ptr(w), _stream()
+            _ptr(z), z.stride(0), _ptr(correction), T, N, groups, keep, top, _ptr(idx), _ptr(w), _stream()
         )
         if rc != 0:
             raise RuntimeError("grouped_topk_route: shape not served")
@@ -1302,6 +1392,96 @@ def routed_combine(
         il = idx.long()
         rows = torch.where(il < experts, il * T + tok, torch.full_like(il, -1))
     return torch_ref.routed_combine(ye, x, rows, w)
+
+
+def residual_routed_add(
+    x: torch.Tensor, y: torch.Tensor, ye: Optional[torch.Tensor] = None,
+    w: Optional[torch.Tensor] = None, rows: Optional[torch.Tensor] = None,
+    idx: Optional[torch.Tensor] = None, experts: int = 0,
+) -> torch.Tensor:
+    """x += y + sum_k w[t, k] ye[row(t, k)] on the fp32 residual x [R, W], in
+    place; returns the new x rounded to y's dtype (x itself when that is
+    fp32).  Rows of ye as in `routed_combine`: a table `rows` int64 [R, top]
+    (all >= 0), or idx * R + t from the choices idx int32 when every expert
+    saw every token.  Without ye only y is added."""
+    R, W = x.shape
+    assert x.dtype == torch.float32 and y.shape == x.shape
+    if ye is not None:
+        assert ye.dim() == 2 and ye.shape[1] == W and ye.dtype == y.dtype
+        assert w.dtype == torch.float32 and w.dim() == 2 and w.shape[0] == R
+        if rows is None:
+            assert idx.dtype == torch.int32 and idx.shape == w.shape and ye.shape[0] == experts * R
+        else:
+            assert rows.dtype == torch.int64 and rows.shape == w.shape
+    if _use_hybrid(x):
+        for t in (x, y, ye, w, rows, idx):
+            assert t is None or t.is_contiguous()
+        xt = None if y.dtype == torch.float32 else torch.empty_like(y)
+        _hl().lig_residual_routed_add(
+            _ptr(x), _ptr(xt), _ptr(y), _ptr(ye), _ptr(rows), _ptr(idx) if rows is None else None,
+            _ptr(w), R, w.shape[1] if w is not None else 0, W, _is_f32(y), _stream(),
+        )
+        return x if xt is None else xt
+    if ye is not None and rows is None:
+        rows = idx.long() * R + torch.arange(R, device=x.device).unsqueeze(1)
+    return torch_ref.residual_routed_add(x, y, ye, w, rows)
+
+
+def small_projection(h: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """h [R, C] times w [N, C] transposed, result in fp32 whatever the storage
+    type: router logits and recurrence gates.  bf16 rows on the GPU with C a
+    multiple of 8 run one MFMA kernel; everything else is an fp32 product."""
+    if _use_hybrid(h) and h.dtype == torch.bfloat16 and h.shape[1] % 8 == 0:
+        assert h.is_contiguous() and w.is_contiguous() and w.dtype == h.dtype
+        R, C = h.shape
+        assert w.shape[1] == C
+        out = torch.empty(R, w.shape[0], dtype=torch.float32, device=h.device)
+        rc = _hl().lig_small_projection(_ptr(out), _ptr(h), _ptr(w), R, w.shape[0], C, _stream())
+        if rc != 0:
+            raise RuntimeError("small_projection: alignment not served")
+        return out
+    return torch.nn.functional.linear(h.float(), w.float())
+
+
+# -- layer norms fused with what enters the residual --------------------------------------
+
+def _layer_norm(x, h, table, tokens, scale, y, w_y, w, eps) -> None:
+    R, H = x.shape
+    for t in (x, h, table, y, w_y, w, tokens):
+        assert t is None or t.is_contiguous()
+    rc = _hl().lig_layer_norm(
+        _ptr(x), _ptr(h), _ptr(table), _ptr(tokens), float(scale), _ptr(y), _ptr(w_y), _ptr(w),
+        float(eps), R, H, _is_f32(w), _stream(),
+    )
+    if rc != 0:
+        raise RuntimeError(f"layer norm: rows of {H} entries not served")
+
+
+def embed_layer_norm(tokens, table, scale: float, w, eps: float):
+    """x = scale * table[token] (fp32, a new residual) and h = LN(x) * w in
+    w's dtype, LN the centred layer norm without bias.  Returns (x, h)."""
+    if _use_hybrid(table):
+        R, H = tokens.shape[0], table.shape[1]
+        assert tokens.dtype == torch.int64 and w.shape == (H,) and w.dtype == table.dtype
+        x = torch.empty(R, H, dtype=torch.float32, device=table.device)
+        h = torch.empty(R, H, dtype=w.dtype, device=table.device)
+        _layer_norm(x, h, table, tokens, scale, None, None, w, eps)
+        return x, h
+    return torch_ref.embed_layer_norm(tokens, table, scale, w, eps)
+
+
+def add_layer_norm(x, w, eps: float, y=None, w_y=None):
+    """With y: x += y / rms(y) * w_y on the fp32 residual, in place.  Returns
+    h = LN(x) * w in w's dtype."""
+    assert x.dtype == torch.float32 and (y is None) == (w_y is None)
+    if _use_hybrid(x):
+        H = x.shape[1]
+        assert w.shape == (H,) and (y is None or (y.shape == x.shape and y.dtype == w.dtype))
+        assert w_y is None or (w_y.shape == (H,) and w_y.dtype == w.dtype)
+        h = torch.empty(x.shape, dtype=w.dtype, device=x.device)
+        _layer_norm(x, h, None, None, 1.0, y, w_y, w, eps)
+        return h
+    return torch_ref.add_layer_norm(x, w, eps, y, w_y)
 
 
 _GLU_KINDS = {"relu": 0, "clamped": 1}

@@ -21,7 +21,9 @@
 // different rows spread over all banks.  The loads of the next tile are
 // issued before the current tile's arithmetic (one tile in registers).
 // Scores, running max and sum are fp32; an optional per-head sink starts a
-// row's running max at sink_h and its sum at one.
+// row's running max at sink_h and its sum at one; an optional gate multiplies
+// the (token, head) output row by one sigmoid (it commutes with whatever
+// linear map per head follows).
 //
 // Grid = (ceil(max segment rows / 64), segments, splits); workgroups past a
 // segment's last row exit at once.  With splits > 1 (few rows, long
@@ -66,6 +68,7 @@ __global__ __launch_bounds__(256) void latent_attention_rows_kernel(
     const uint16_t* __restrict__ q,      // [R, H * D] contiguous
     const uint16_t* __restrict__ cache,  // [blocks, 1, BS, D]
     const float* __restrict__ sink,      // nullable, [H]
+    const uint16_t* __restrict__ gate, long gate_stride,  // nullable, [R, H] pre-sigmoid
     const int* __restrict__ seg_start, const int* __restrict__ seg_len,
     const int* __restrict__ seg_ctx,     // tokens of the sequence after this step
     const int* __restrict__ block_tables, int max_blocks, float scale, int H,
@@ -301,6 +304,10 @@ __global__ __launch_bounds__(256) void latent_attention_rows_kernel(
     const long orho = rho0 + wave * 16 + lg * 4 + r;
     if (orho >= nrows) continue;
     uint16_t* op = out + ((size_t)lo * H + orho) * Dv;
+    if (gate != nullptr) {
+      const long ot = orho / H;
+      inv_l[r] *= sigmoid_fast(bf16_to_f32(gate[(lo + ot) * gate_stride + (orho - ot * H)]));
+    }
 #pragma unroll
     for (int db = 0; db < DB; ++db) {
       const int d = db * 16 + li;
@@ -317,7 +324,7 @@ __global__ __launch_bounds__(256) void latent_attention_rows_kernel(
 // to Dv + 4 floats so that they stay 16-byte aligned).
 __global__ __launch_bounds__(256) void latent_attention_rows_combine_kernel(
     uint16_t* __restrict__ out, const float* __restrict__ partial,
-    const int* __restrict__ seg_start, const int* __restrict__ seg_len, int H,
+    const uint16_t* __restrict__ gate, long gate_stride, const int* __restrict__ seg_start, const int* __restrict__ seg_len, int H,
     int Dv, int nsplit) {
   const int s = blockIdx.y;
   const long nrows = (long)seg_len[s] * H;
@@ -335,7 +342,11 @@ __global__ __launch_bounds__(256) void latent_attention_rows_combine_kernel(
   const float mstar = wave_reduce_max(mz);
   const float wz = (mz == -INFINITY) ? 0.f : __expf(mz - mstar);
   const float lsum = wave_reduce_sum(wz * lz);
-  const float inv = lsum > 0.f ? 1.0f / lsum : 0.f;
+  float inv = lsum > 0.f ? 1.0f / lsum : 0.f;
+  if (gate != nullptr) {
+    const long tok = rho / H;
+    inv *= sigmoid_fast(bf16_to_f32(gate[(seg_start[s] + tok) * gate_stride + (rho - tok * H)]));
+  }
   for (int d0 = 0; d0 < Dv; d0 += 256) {  // uniform trip count: every lane feeds the shuffles
     const int d = d0 + lane * 4;
     const bool act = d < Dv;
@@ -375,6 +386,7 @@ __global__ __launch_bounds__(256) void latent_attention_rows_combine_kernel(
 // uses another kernel).
 extern "C" int lig_latent_attention_rows(
     void* out, const void* q, const void* cache, const float* sink,
+    const void* gate, long gate_stride,
     const int* seg_start, const int* seg_len, const int* seg_ctx,
     const int* block_tables, int max_blocks, float scale, int num_segs,
     int max_seg_len, int H, int D, int Dv, int block_size, int nsplit,
@@ -391,7 +403,8 @@ extern "C" int lig_latent_attention_rows(
 #define LAUNCH_LR(DKP, DVP)                                                    \
   hipLaunchKernelGGL((latent_attention_rows_kernel<DKP, DVP>), grid, block, 0, \
                      stream, (uint16_t*)out, (const uint16_t*)q,               \
-                     (const uint16_t*)cache, sink, seg_start, seg_len,         \
+                     (const uint16_t*)cache, sink,                             \
+                     (const uint16_t*)gate, gate_stride, seg_start, seg_len,         \
                      seg_ctx, block_tables, max_blocks, scale, H, D, Dv,       \
                      block_size, nsplit, partial)
   if (D <= 64 && Dv <= 64) LAUNCH_LR(64, 64);
@@ -405,7 +418,7 @@ extern "C" int lig_latent_attention_rows(
     const long rows4 = ((long)max_seg_len * H + 3) / 4;
     hipLaunchKernelGGL(latent_attention_rows_combine_kernel,
                        dim3((unsigned)rows4, num_segs), dim3(256), 0, stream,
-                       (uint16_t*)out, partial, seg_start, seg_len, H, Dv, nsplit);
+                       (uint16_t*)out, partial, (const uint16_t*)gate, gate_stride, seg_start, seg_len, H, Dv, nsplit);
   }
   return 0;
 }

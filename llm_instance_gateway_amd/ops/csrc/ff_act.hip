@@ -1,4 +1,5 @@
-// Feed-forward activations between the two GEMMs, gfx950: squared ReLU, the
+// Feed-forward activations between the two GEMMs, gfx950: squared ReLU (also
+// between column blocks of wider rows), the tanh-gelu times a gathered table row, the
 // gated SiLU (silu(gate) * up over a fused [gate | up] projection), the exact
 // (erf) gelu, tanh, and the tanh soft cap of fp32 logits.
 // fp32 arithmetic, bf16 or fp32 storage; 4-element vectors when the row
@@ -16,6 +17,46 @@ __global__ void relu_squared_kernel(T* __restrict__ out, const T* __restrict__ x
     for (int k = 0; k < N; ++k) {
       const float z = fmaxf(v[k], 0.f);
       v[k] = z * z;
+    }
+    stn<N>(out + i, v);
+  }
+}
+
+// Column blocks of F entries inside wider rows.
+template <typename T, int N>
+__global__ void relu_squared_rows_kernel(T* __restrict__ out, long out_stride,
+                                         const T* __restrict__ x, long x_stride, int F, long n) {
+  for (long i = (blockIdx.x * (long)blockDim.x + threadIdx.x) * N; i < n;
+       i += gridDim.x * (long)blockDim.x * N) {
+    const long r = i / F;
+    const int c = (int)(i - r * F);
+    float v[N];
+    ldn<N>(x + r * x_stride + c, v);
+#pragma unroll
+    for (int k = 0; k < N; ++k) {
+      const float z = fmaxf(v[k], 0.f);
+      v[k] = z * z;
+    }
+    stn<N>(out + r * out_stride + c, v);
+  }
+}
+
+// out[r] = gelu_tanh(z[r]) * table[tokens[r], col : col + F]
+template <typename T, int N>
+__global__ void gelu_tanh_table_mul_kernel(T* __restrict__ out, const T* __restrict__ z,
+                                           const T* __restrict__ table, long table_stride,
+                                           const int64_t* __restrict__ tokens, int F, long n) {
+  for (long i = (blockIdx.x * (long)blockDim.x + threadIdx.x) * N; i < n;
+       i += gridDim.x * (long)blockDim.x * N) {
+    const long r = i / F;
+    const int c = (int)(i - r * F);
+    float v[N], e[N];
+    ldn<N>(z + i, v);
+    ldn<N>(table + tokens[r] * table_stride + c, e);
+#pragma unroll
+    for (int k = 0; k < N; ++k) {
+      const float a = v[k];
+      v[k] = 0.5f * a * (1.0f + tanhf(0.79788456080286535588f * (a + 0.044715f * a * a * a))) * e[k];
     }
     stn<N>(out + i, v);
   }
@@ -107,6 +148,43 @@ void lig_relu_squared(void* out, const void* x, long n, int is_f32, hipStream_t 
     if (v4) LIG_R2(bf16s, 4); else LIG_R2(bf16s, 1);
   }
 #undef LIG_R2
+}
+
+void lig_relu_squared_rows(void* out, long out_stride, const void* x, long x_stride, long rows,
+                           int F, int is_f32, hipStream_t s) {
+  const long n = rows * F;
+  if (n <= 0) return;
+  const bool v4 = F % 4 == 0 && out_stride % 4 == 0 && x_stride % 4 == 0 && aligned16(out) && aligned16(x);
+  long g = ((v4 ? n / 4 : n) + 255) / 256;
+  const int grid = (int)(g > 65535 ? 65535 : g);
+#define LIG_R2(T, N)                                                                \
+  hipLaunchKernelGGL((relu_squared_rows_kernel<T, N>), dim3(grid), dim3(256), 0, s, \
+                     (T*)out, out_stride, (const T*)x, x_stride, F, n)
+  if (is_f32) {
+    if (v4) LIG_R2(float, 4); else LIG_R2(float, 1);
+  } else {
+    if (v4) LIG_R2(bf16s, 4); else LIG_R2(bf16s, 1);
+  }
+#undef LIG_R2
+}
+
+void lig_gelu_tanh_table_mul(void* out, const void* z, const void* table, long table_stride,
+                             const int64_t* tokens, long rows, int F, int is_f32,
+                             hipStream_t s) {
+  const long n = rows * F;
+  if (n <= 0) return;
+  const bool v4 = F % 4 == 0 && table_stride % 4 == 0 && aligned16(out) && aligned16(z) && aligned16(table);
+  long g = ((v4 ? n / 4 : n) + 255) / 256;
+  const int grid = (int)(g > 65535 ? 65535 : g);
+#define LIG_GT(T, N)                                                                  \
+  hipLaunchKernelGGL((gelu_tanh_table_mul_kernel<T, N>), dim3(grid), dim3(256), 0, s, \
+                     (T*)out, (const T*)z, (const T*)table, table_stride, tokens, F, n)
+  if (is_f32) {
+    if (v4) LIG_GT(float, 4); else LIG_GT(float, 1);
+  } else {
+    if (v4) LIG_GT(bf16s, 4); else LIG_GT(bf16s, 1);
+  }
+#undef LIG_GT
 }
 
 void lig_silu_mul(void* out, const void* x, long rows, int F, int is_f32,

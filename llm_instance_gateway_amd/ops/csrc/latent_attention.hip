@@ -1,7 +1,8 @@
 // Front end of latent (low-rank key/value) attention, gfx950.
 //
-// One fused projection gives, per token, a query latent, a key/value latent
-// and one rotated key part shared by all heads.  `latent_kv_prep` RMS-norms
+// One fused projection gives, per token, a query latent (none in models that
+// project queries directly: q_rank 0), a key/value latent and one rotated key
+// part shared by all heads.  `latent_kv_prep` RMS-norms
 // both latents (plain weights), rotates the shared key part and writes the
 // token's cache row [normed key/value latent | rotated key part] straight
 // into the paged cache; only that row is ever cached.  `rotate_pack_queries`
@@ -11,6 +12,8 @@
 //
 // Rotation: interleaved pairs (2i, 2i+1), angle = position * inv_freq[i] in
 // fp32, accurate sinf/cosf.  Entries past 2 * n_freq pass unchanged.
+// `rotary_table` tabulates cosines and sines of a step's positions once, for
+// kernels that rotate the same rows in several layers.
 
 #include "elem_types.h"
 
@@ -139,7 +142,7 @@ __global__ __launch_bounds__(LA_THREADS) void latent_kv_prep_vec_kernel(
 template <typename T>
 __global__ void rotate_pack_queries_kernel(
     T* __restrict__ out,       // [R, heads, lead + rot_dim]
-    const T* __restrict__ q,   // [R, heads, dim + rot_dim]
+    const T* __restrict__ q, long q_stride,  // rows of [heads, dim + rot_dim]
     const float* __restrict__ inv_freq, int n_freq,
     const int64_t* __restrict__ positions, int heads, int dim, int rot_dim,
     int lead, long total) {  // total = R * heads * pairs
@@ -149,7 +152,7 @@ __global__ void rotate_pack_queries_kernel(
     const int i = (int)(idx % pairs);
     const long rh = idx / pairs;
     const long r = rh / heads;
-    const T* src = q + rh * (dim + rot_dim) + dim;
+    const T* src = q + r * q_stride + (rh - r * heads) * (dim + rot_dim) + dim;
     T* dst = out + rh * (lead + rot_dim) + lead;
     const int d = 2 * i;
     const float u = ld(src + d);
@@ -175,8 +178,8 @@ __global__ void rotate_pack_queries_kernel(
 // multiples of 8.
 template <typename T>
 __global__ void rotate_pack_queries_vec_kernel(
-    T* __restrict__ out, const T* __restrict__ q, const float* __restrict__ inv_freq,
-    int n_freq, const int64_t* __restrict__ positions, int heads, int dim,
+    T* __restrict__ out, const T* __restrict__ q, long q_stride,
+    const float* __restrict__ inv_freq, int n_freq, const int64_t* __restrict__ positions, int heads, int dim,
     int rot_dim, int lead, long total) {  // total = R * heads * rot_dim / 8
   const int chunks = rot_dim / 8;
   for (long idx = blockIdx.x * (long)blockDim.x + threadIdx.x; idx < total;
@@ -185,7 +188,7 @@ __global__ void rotate_pack_queries_vec_kernel(
     const long rh = idx / chunks;
     const long r = rh / heads;
     float v[8];
-    ld8(q + rh * (dim + rot_dim) + dim + c * 8, v);
+    ld8(q + r * q_stride + (rh - r * heads) * (dim + rot_dim) + dim + c * 8, v);
     const float pos = (float)positions[r];
 #pragma unroll
     for (int k = 0; k < 4; ++k) {
@@ -199,6 +202,19 @@ __global__ void rotate_pack_queries_vec_kernel(
       }
     }
     st8(out + rh * (lead + rot_dim) + lead + c * 8, v);
+  }
+}
+
+// cs[r] = [cos(pos_r * f_i) | sin(pos_r * f_i)], i < n_freq, fp32.
+__global__ void rotary_table_kernel(float* __restrict__ cs, const int64_t* __restrict__ positions,
+                                    const float* __restrict__ inv_freq, int n_freq, long total) {
+  for (long e = blockIdx.x * (long)blockDim.x + threadIdx.x; e < total;
+       e += gridDim.x * (long)blockDim.x) {
+    const long r = e / n_freq;
+    const int i = (int)(e - r * n_freq);
+    const float ang = (float)positions[r] * inv_freq[i];
+    cs[r * 2 * n_freq + i] = cosf(ang);
+    cs[r * 2 * n_freq + n_freq + i] = sinf(ang);
   }
 }
 
@@ -259,22 +275,22 @@ void lig_latent_kv_prep(void* cq_out, const void* proj, long proj_stride,
                        kv_rank, rot_dim);
 }
 
-void lig_rotate_pack_queries(void* out, const void* q, const float* inv_freq,
+void lig_rotate_pack_queries(void* out, const void* q, long q_stride, const float* inv_freq,
                              int n_freq, const int64_t* positions, int R,
                              int heads, int dim, int rot_dim, int lead,
                              int is_f32, hipStream_t s) {
-  if (dim % 8 == 0 && rot_dim % 8 == 0 && lead % 8 == 0 && aligned16(out) && aligned16(q)) {
+  if (dim % 8 == 0 && rot_dim % 8 == 0 && lead % 8 == 0 && q_stride % 8 == 0 && aligned16(out) && aligned16(q)) {
     const long total8 = (long)R * heads * (rot_dim / 8);
     if (total8 <= 0) return;
     long g8 = (total8 + 255) / 256;
     const int grid8 = (int)(g8 > 65535 ? 65535 : g8);
     if (is_f32)
       hipLaunchKernelGGL(rotate_pack_queries_vec_kernel<float>, dim3(grid8), dim3(256), 0, s,
-                         (float*)out, (const float*)q, inv_freq, n_freq, positions,
+                         (float*)out, (const float*)q, q_stride, inv_freq, n_freq, positions,
                          heads, dim, rot_dim, lead, total8);
     else
       hipLaunchKernelGGL(rotate_pack_queries_vec_kernel<bf16s>, dim3(grid8), dim3(256), 0, s,
-                         (bf16s*)out, (const bf16s*)q, inv_freq, n_freq, positions,
+                         (bf16s*)out, (const bf16s*)q, q_stride, inv_freq, n_freq, positions,
                          heads, dim, rot_dim, lead, total8);
     return;
   }
@@ -284,12 +300,22 @@ void lig_rotate_pack_queries(void* out, const void* q, const float* inv_freq,
   const int grid = (int)(g > 65535 ? 65535 : g);
   if (is_f32)
     hipLaunchKernelGGL(rotate_pack_queries_kernel<float>, dim3(grid), dim3(256), 0, s,
-                       (float*)out, (const float*)q, inv_freq, n_freq, positions,
+                       (float*)out, (const float*)q, q_stride, inv_freq, n_freq, positions,
                        heads, dim, rot_dim, lead, total);
   else
     hipLaunchKernelGGL(rotate_pack_queries_kernel<bf16s>, dim3(grid), dim3(256), 0, s,
-                       (bf16s*)out, (const bf16s*)q, inv_freq, n_freq, positions,
+                       (bf16s*)out, (const bf16s*)q, q_stride, inv_freq, n_freq, positions,
                        heads, dim, rot_dim, lead, total);
+}
+
+void lig_rotary_table(float* cs, const int64_t* positions, const float* inv_freq, int R,
+                      int n_freq, hipStream_t s) {
+  const long total = (long)R * n_freq;
+  if (total <= 0) return;
+  long g = (total + 255) / 256;
+  const int grid = (int)(g > 65535 ? 65535 : g);
+  hipLaunchKernelGGL(rotary_table_kernel, dim3(grid), dim3(256), 0, s, cs, positions,
+                     inv_freq, n_freq, total);
 }
 
 void lig_scale_gather_rows(void* out, const void* x, const int64_t* idx,

@@ -7,23 +7,36 @@
 //   constant-decay form (one d per head):
 //       S  <- d S + k_t v_t^T
 //       o_t = S^T q_t
-//   optional silu on q, k, v as they are read.
+//   gated form (one log input gate i and log forget gate f per head and
+//   token, both squashed by cap * tanh(. / cap), f through log-sigmoid):
+//       m_t = max(f + m_{t-1}, i)            (m starts at 0)
+//       S_t = exp(f + m_{t-1} - m_t) S_{t-1} + exp(i - m_t) k_t v_t^T
+//       n_t likewise with k_t alone
+//       o_t = S_t^T q_t / (max(|n_t . q_t|, exp(-m_t)) + 1e-6)
+//   optional on q and k as they are read: silu (also on v), a rotate-half
+//   rotation by tabulated cosines and sines, a constant factor each.
 //
-// One workgroup per (segment, head).  A thread owns value column j and one
-// SPLIT-th of the key channels (lane = SPLIT j + s, keys s*KPT .. s*KPT +
-// KPT-1, KPT one of a few size classes; SPLIT is 8 for heads of 32 or more
-// key channels when 8 Dv threads fit a workgroup, else 4), keeps its KPT
-// state entries in registers for the whole segment, and the partial outputs
-// of a column are summed with lane shuffles.  The
-// segment is walked serially, TT (8 to 32) tokens staged into LDS at a time (q, k, the
-// decay already exponentiated, v), so a prompt portion and a single decoded
-// token take the same arithmetic path in the same order: results do not
-// depend on how a sequence is cut into steps.
+// One workgroup per (segment, head, block of up to 64 value columns).  A
+// thread owns value column j of the block and one SPLIT-th of the key
+// channels (lane = SPLIT j + s, keys s*KPT .. s*KPT + KPT-1, KPT one of a few
+// size classes; SPLIT is 8 for heads of 32 or more key channels, else 4),
+// keeps its KPT state entries in registers for the whole segment, and the
+// partial outputs of a column are summed with lane permutes.  In the gated
+// form the vector n is one more column of every block whose value is 1, so
+// n . q falls out of the same walk; outputs wait in LDS until the tile ends
+// and are divided on their way out.  The segment is walked serially, TT (8
+// to 32) tokens staged into LDS at a time (q, k, decays and gates already
+// exponentiated, v), so a prompt portion and a single decoded token take the
+// same arithmetic path in the same order: results do not depend on how a
+// sequence is cut into steps.  (The running maximum inside a tile comes from
+// a prefix sum and a prefix maximum over the lanes; it is only the scale S
+// and n are kept at, and both decays are taken from the very values of m
+// that are stored.)
 //
 // The state row of a sequence is stored in the order the threads hold it,
-// [head][ii][thread] with D padded to SPLIT*KPT: loads and stores are
-// coalesced (a row holds H * SPLIT * KPT * Dv entries; ops.matrix_state_width
-// mirrors this).
+// [head][block][ii][thread] with D padded to SPLIT*KPT: loads and stores are
+// coalesced; in the gated form the running maxima [head][block] follow
+// (ops.matrix_state_width mirrors this).
 // A segment that starts its sequence ignores what the slot held.
 
 #include "elem_types.h"
@@ -46,47 +59,94 @@ LIG_DEVICE float split_sum(float o) {
   return o;
 }
 
+#define MS_COLS 64  // value columns per workgroup
+
+enum { MS_CONST = 0, MS_BONUS = 1, MS_GATED = 2 };
+
+struct MsArgs {
+  float* out;  // [R, H*Dv]
+  const void *q, *k, *v;
+  long q_stride, k_stride, v_stride;
+  const float* decay_pre;   // [R, H*D]   (bonus form)
+  const float* head_decay;  // [H]        (constant form)
+  const float* bonus;       // [H*D]      (bonus form)
+  const float *gate_i, *gate_f;  // [R, H] views, row stride gate_stride (gated form)
+  long gate_stride;
+  const float *bias_i, *bias_f;  // [H]
+  float gate_cap;
+  const float* cs;  // nullable: [R, 2*nf] cosines | sines of the rotation
+  int nf;
+  float q_scale, k_scale;
+  float* state;
+  long state_stride;
+  const int *seg_start, *seg_len, *seg_slot, *seg_fresh;
+  int H, D, Dv, CB, NB, TT, act_silu;
+};
+
+// Entry i of a query or key head as the recurrence sees it: silu, rotation
+// (entry i paired with i +- nf), constant factor; fp32 throughout.
+template <typename T>
+LIG_DEVICE float ms_prep(const T* __restrict__ x, int i, const float* __restrict__ cs, int nf,
+                         float scale, int act_silu) {
+  float a = ld(x + i);
+  if (act_silu) a = a * sigmoid_f32(a);
+  if (i < 2 * nf) {
+    const bool lower = i < nf;
+    const int p = lower ? i : i - nf;
+    float b = ld(x + (lower ? i + nf : i - nf));
+    if (act_silu) b = b * sigmoid_f32(b);
+    const float c = cs[p], s = cs[nf + p];
+    a = lower ? a * c - b * s : a * c + b * s;
+  }
+  return a * scale;
+}
+
 // KPT: key channels per thread (D is padded to SPLIT * KPT; padded channels carry
-// q = k = w = 0 and stay zero).  MAXT bounds the workgroup size (4 * Dv
-// rounded up to whole waves) so the compiler may use the register file a
-// small workgroup leaves it.
-template <typename T, int MS_SPLIT, int KPT, bool BONUS, int MAXT>
-__global__ __launch_bounds__(MAXT) void matrix_state_scan_kernel(
-    float* __restrict__ out,  // [R, H*Dv]
-    const T* __restrict__ q, long q_stride, const T* __restrict__ k, long k_stride,
-    const T* __restrict__ v, long v_stride,
-    const float* __restrict__ decay_pre,   // [R, H*D]   (BONUS)
-    const float* __restrict__ head_decay,  // [H]        (!BONUS)
-    const float* __restrict__ bonus,       // [H*D]      (BONUS)
-    float* __restrict__ state, long state_stride, const int* __restrict__ seg_start,
-    const int* __restrict__ seg_len, const int* __restrict__ seg_slot,
-    const int* __restrict__ seg_fresh, int H, int D, int Dv, int TT, int act_silu) {
+// q = k = w = 0 and stay zero).  MAXT bounds the workgroup size (SPLIT times
+// the block's columns rounded up to whole waves) so the compiler may use the
+// register file a small workgroup leaves it.
+template <typename T, int MS_SPLIT, int KPT, int FORM, int MAXT>
+__global__ __launch_bounds__(MAXT) void matrix_state_scan_kernel(const MsArgs A) {
   extern __shared__ __align__(16) float sm[];
+  constexpr bool BONUS = FORM == MS_BONUS, GATED = FORM == MS_GATED;
   constexpr int Dp = MS_SPLIT * KPT;
+  const int H = A.H, D = A.D, Dv = A.Dv, TT = A.TT;
+  const int CBw = GATED ? A.CB + 1 : A.CB;  // columns that own state
   float* q_s = sm;                 // [TT][Dp]
   float* k_s = q_s + TT * Dp;      // [TT][Dp]
   float* w_s = k_s + TT * Dp;      // [TT][Dp] (BONUS only)
-  float* v_s = BONUS ? w_s + TT * Dp : w_s;  // [TT][Dv]
+  float* v_s = BONUS ? w_s + TT * Dp : w_s;  // [TT][CBw]
+  float* o_s = v_s + TT * CBw;     // [TT][CBw] (GATED only), then
+  float* a_s = o_s + TT * CBw;     // [TT] kept share of the state,
+  float* b_s = a_s + TT;           // [TT] weight of the new key,
+  float* e_s = b_s + TT;           // [TT] exp(-m)
 
-  const int seg = blockIdx.x, h = blockIdx.y;
-  const int n = seg_len[seg];
+  const int seg = blockIdx.x, h = blockIdx.y, blk = blockIdx.z;
+  const int n = A.seg_len[seg];
   if (n <= 0) return;
-  const int r0 = seg_start[seg];
+  const int r0 = A.seg_start[seg];
   const int tid = threadIdx.x, nt = blockDim.x;
   const int j = tid / MS_SPLIT, s = tid % MS_SPLIT;
-  const bool owner = j < Dv;
-  const int nthr = Dv * MS_SPLIT;  // threads that own state
+  const bool owner = j < CBw;
+  const int nthr = CBw * MS_SPLIT;  // threads that own state
+  const int c0 = blk * A.CB, ncol = min(A.CB, Dv - c0);
+  const T* q = (const T*)A.q + h * D;
+  const T* k = (const T*)A.k + h * D;
+  const T* v = (const T*)A.v + h * Dv + c0;
 
   float S[KPT], U[KPT];
-  float* srow = state + (long)seg_slot[seg] * state_stride + (long)h * KPT * nthr;
-  const bool load_state = owner && seg_fresh[seg] == 0;
+  float* slot = A.state + (long)A.seg_slot[seg] * A.state_stride;
+  float* srow = slot + (long)(h * A.NB + blk) * KPT * nthr;
+  float* mrow = slot + (long)H * A.NB * KPT * nthr + h * A.NB + blk;  // (GATED)
+  const bool resume = A.seg_fresh[seg] == 0;
 #pragma unroll
   for (int ii = 0; ii < KPT; ++ii) {
-    S[ii] = load_state ? srow[(long)ii * nthr + tid] : 0.f;
+    S[ii] = (owner && resume) ? srow[(long)ii * nthr + tid] : 0.f;
     const int i = s * KPT + ii;
-    U[ii] = (BONUS && i < D) ? bonus[h * D + i] : 0.f;
+    U[ii] = (BONUS && i < D) ? A.bonus[h * D + i] : 0.f;
   }
-  const float dconst = BONUS ? 0.f : head_decay[h];
+  const float dconst = FORM == MS_CONST ? A.head_decay[h] : 0.f;
+  float m_run = (GATED && resume) ? *mrow : 0.f;  // wave 0 carries it along
 
 #pragma nounroll
   for (int t0 = 0; t0 < n; t0 += TT) {
@@ -98,31 +158,65 @@ __global__ __launch_bounds__(MAXT) void matrix_state_scan_kernel(
       const long r = r0 + t0 + t;
       float qv = 0.f, kv = 0.f, wv = 0.f;
       if (i < D) {
-        qv = ld(q + r * q_stride + h * D + i);
-        kv = ld(k + r * k_stride + h * D + i);
-        if (act_silu) {
-          qv = qv * sigmoid_f32(qv);
-          kv = kv * sigmoid_f32(kv);
-        }
-        if (BONUS) wv = expf(-expf(decay_pre[r * (long)(H * D) + h * D + i]));
+        const float* cs = A.cs + r * 2 * A.nf;
+        qv = ms_prep(q + r * A.q_stride, i, cs, A.nf, A.q_scale, A.act_silu);
+        kv = ms_prep(k + r * A.k_stride, i, cs, A.nf, A.k_scale, A.act_silu);
+        if (BONUS) wv = expf(-expf(A.decay_pre[r * (long)(H * D) + h * D + i]));
       }
       q_s[e] = qv;
       k_s[e] = kv;
       if (BONUS) w_s[e] = wv;
     }
 #pragma nounroll
-    for (int e = tid; e < nt_tok * Dv; e += nt) {
-      const int t = e / Dv, c = e - t * Dv;
-      float vv = ld(v + (long)(r0 + t0 + t) * v_stride + h * Dv + c);
-      if (act_silu) vv = vv * sigmoid_f32(vv);
+    for (int e = tid; e < nt_tok * CBw; e += nt) {
+      const int t = e / CBw, c = e - t * CBw;
+      float vv = (GATED && c == A.CB) ? 1.0f : 0.f;
+      if (c < ncol) {
+        vv = ld(v + (long)(r0 + t0 + t) * A.v_stride + c);
+        if (A.act_silu) vv = vv * sigmoid_f32(vv);
+      }
       v_s[e] = vv;
+    }
+    if (GATED && tid < WAVE_SIZE) {
+      // lane t: gates of token t, prefix sum of the log forget gates, prefix
+      // maximum of (i - that sum)
+      float gi = -INFINITY, gf = 0.f;
+      if (tid < nt_tok) {
+        const long r = (long)(r0 + t0 + tid) * A.gate_stride + h;
+        gi = A.gate_cap * tanhf((A.gate_i[r] + A.bias_i[h]) / A.gate_cap);
+        gf = A.gate_cap * tanhf((A.gate_f[r] + A.bias_f[h]) / A.gate_cap);
+        gf = fminf(gf, 0.f) - log1pf(expf(-fabsf(gf)));
+      }
+      float F = gf;
+#pragma unroll
+      for (int d = 1; d < 32; d <<= 1) {
+        const float u = __shfl_up(F, d, WAVE_SIZE);
+        if (tid >= d) F += u;
+      }
+      float G = gi - F;
+#pragma unroll
+      for (int d = 1; d < 32; d <<= 1) {
+        const float u = __shfl_up(G, d, WAVE_SIZE);
+        if (tid >= d) G = fmaxf(G, u);
+      }
+      const float m = F + fmaxf(m_run, G);
+      float m_prev = __shfl_up(m, 1, WAVE_SIZE);
+      if (tid == 0) m_prev = m_run;
+      if (tid < nt_tok) {
+        a_s[tid] = expf(gf + m_prev - m);
+        b_s[tid] = expf(gi - m);
+        e_s[tid] = expf(-m);
+      }
+      m_run = __shfl(m, nt_tok - 1, WAVE_SIZE);
     }
     __syncthreads();
     // every wave of the workgroup walks the tile (idle lanes of the last
     // wave take part in the lane permutes with zeros)
     // one token: read its q, k, decay and v from LDS, output, state update
     auto step = [&](int t) __attribute__((always_inline)) {
-      const float vj = owner ? v_s[t * Dv + j] : 0.f;
+      float vj = owner ? v_s[t * CBw + j] : 0.f;
+      const float keep = GATED ? a_s[t] : dconst;
+      if (GATED) vj *= b_s[t];
       const float* qt = q_s + t * Dp + s * KPT;
       const float* kt = k_s + t * Dp + s * KPT;
       const float* wt = w_s + t * Dp + s * KPT;
@@ -141,13 +235,16 @@ __global__ __launch_bounds__(MAXT) void matrix_state_scan_kernel(
             o += q4[e] * (S[ii] + U[ii] * kv);
             S[ii] = w4[e] * S[ii] + kv;
           } else {
-            S[ii] = dconst * S[ii] + kv;
+            S[ii] = keep * S[ii] + kv;
             o += q4[e] * S[ii];
           }
         }
       }
       o = split_sum<MS_SPLIT>(o);
-      if (owner && s == 0) out[(long)(r0 + t0 + t) * (H * Dv) + h * Dv + j] = o;
+      if (owner && s == 0) {
+        if (GATED) o_s[t * CBw + j] = o;
+        else if (j < ncol) A.out[(long)(r0 + t0 + t) * (H * Dv) + h * Dv + c0 + j] = o;
+      }
     };
     // two tokens per trip: the second token's LDS reads overlap the first
     // token's arithmetic (the state update itself stays in order)
@@ -158,19 +255,28 @@ __global__ __launch_bounds__(MAXT) void matrix_state_scan_kernel(
       step(t + 1);
     }
     if (t < nt_tok) step(t);
+    if (GATED) {
+      __syncthreads();
+#pragma nounroll
+      for (int e = tid; e < nt_tok * ncol; e += nt) {
+        const int tt = e / ncol, c = e - tt * ncol;
+        const float den = fmaxf(fabsf(o_s[tt * CBw + A.CB]), e_s[tt]) + 1e-6f;
+        A.out[(long)(r0 + t0 + tt) * (H * Dv) + h * Dv + c0 + c] = o_s[tt * CBw + c] / den;
+      }
+    }
   }
   if (owner) {
 #pragma unroll
     for (int ii = 0; ii < KPT; ++ii) srow[(long)ii * nthr + tid] = S[ii];
   }
+  if (GATED && tid == 0) *mrow = m_run;
 }
 
-// Key split and key channels per thread for a head of D key channels and Dv
-// value channels: the smallest size class that holds ceil(D / split); kpt 0
-// when D is too wide.
-static void ms_shape(int D, int Dv, int* split, int* kpt) {
+// Key split and key channels per thread for a head of D key channels: the
+// smallest size class that holds ceil(D / split); kpt 0 when D is too wide.
+static void ms_shape(int D, int* split, int* kpt) {
   static const int classes[] = {4, 8, 12, 16, 24, 32, 48, 64};
-  *split = (D >= 32 && Dv * 8 <= 1024) ? 8 : 4;
+  *split = D >= 32 ? 8 : 4;
   const int need = (D + *split - 1) / *split;
   *kpt = 0;
   for (int c : classes)
@@ -180,65 +286,77 @@ static void ms_shape(int D, int Dv, int* split, int* kpt) {
     }
 }
 
-// Returns 0 when launched, 1 when a head is wider than the kernel holds.
+template <typename T, int SPLIT, int KPT, int FORM>
+static void ms_launch(const MsArgs& a, dim3 grid, int threads, size_t smem, hipStream_t stream) {
+  if (threads <= 256)
+    hipLaunchKernelGGL((matrix_state_scan_kernel<T, SPLIT, KPT, FORM, 256>), grid,
+                       dim3(threads), smem, stream, a);
+  else
+    hipLaunchKernelGGL((matrix_state_scan_kernel<T, SPLIT, KPT, FORM, 576>), grid,
+                       dim3(threads), smem, stream, a);
+}
+
+template <typename T, int FORM>
+static void ms_dispatch(const MsArgs& a, int split, int kpt, dim3 grid, int threads,
+                        size_t smem, hipStream_t st) {
+  if (split == 4) {
+    if (kpt == 4) ms_launch<T, 4, 4, FORM>(a, grid, threads, smem, st);
+    else ms_launch<T, 4, 8, FORM>(a, grid, threads, smem, st);
+    return;
+  }
+  switch (kpt) {
+    case 4: ms_launch<T, 8, 4, FORM>(a, grid, threads, smem, st); break;
+    case 8: ms_launch<T, 8, 8, FORM>(a, grid, threads, smem, st); break;
+    case 12: ms_launch<T, 8, 12, FORM>(a, grid, threads, smem, st); break;
+    case 16: ms_launch<T, 8, 16, FORM>(a, grid, threads, smem, st); break;
+    case 24: ms_launch<T, 8, 24, FORM>(a, grid, threads, smem, st); break;
+    case 32: ms_launch<T, 8, 32, FORM>(a, grid, threads, smem, st); break;
+    case 48: ms_launch<T, 8, 48, FORM>(a, grid, threads, smem, st); break;
+    default: ms_launch<T, 8, 64, FORM>(a, grid, threads, smem, st); break;
+  }
+}
+
+// The form follows from the pointers: bonus -> bonus form, gate_i -> gated
+// form, else the constant-decay form.  Returns 0 when launched, 1 when a head
+// is wider than the kernel holds.
 extern "C" int lig_matrix_state_scan(
     float* out, const void* q, long q_stride, const void* k, long k_stride,
     const void* v, long v_stride, const float* decay_pre, const float* head_decay,
-    const float* bonus, float* state, long state_stride, const int* seg_start,
+    const float* bonus, const float* gate_i, const float* gate_f, long gate_stride,
+    const float* bias_i, const float* bias_f, float gate_cap, const float* cs, int nf,
+    float q_scale, float k_scale, float* state, long state_stride, const int* seg_start,
     const int* seg_len, const int* seg_slot, const int* seg_fresh, int S, int H,
     int D, int Dv, int act_silu, int is_f32, hipStream_t stream) {
   int split = 4, kpt = 0;
-  if (D > 0) ms_shape(D, Dv, &split, &kpt);
-  if (kpt == 0 || Dv <= 0 || Dv > 256) return 1;
+  if (D > 0) ms_shape(D, &split, &kpt);
+  if (kpt == 0 || Dv <= 0 || 2 * nf > D) return 1;
+  const int CB = Dv < MS_COLS ? Dv : MS_COLS;
+  const int NB = (Dv + CB - 1) / CB;
+  if (H > 65535 || NB > 65535) return 1;
   if (S <= 0) return 0;
+  const int form = bonus != nullptr ? MS_BONUS : (gate_i != nullptr ? MS_GATED : MS_CONST);
+  const int CBw = form == MS_GATED ? CB + 1 : CB;
   const int Dp = kpt * split;
-  const bool has_bonus = bonus != nullptr;
-  const int per_tok = (has_bonus ? 3 : 2) * Dp + Dv;
+  const int per_tok = (form == MS_BONUS ? 3 : 2) * Dp + (form == MS_GATED ? 2 * CBw + 3 : CBw);
   // tokens staged per tile: as many as 40 KB of LDS hold, 8 to 32
   const int TT = per_tok * 32 * 4 <= 40 * 1024 ? 32 : (per_tok * 16 * 4 <= 48 * 1024 ? 16 : 8);
   const size_t smem = (size_t)per_tok * TT * sizeof(float);
-  const int threads = ((Dv * split + WAVE_SIZE - 1) / WAVE_SIZE) * WAVE_SIZE;
-  dim3 grid(S, H), block(threads);
-#define LIG_MS_T(T, SP, KPT, B, MAXT)                                           \
-  hipLaunchKernelGGL((matrix_state_scan_kernel<T, SP, KPT, B, MAXT>), grid,     \
-                     block, smem, stream, out, (const T*)q, q_stride,           \
-                     (const T*)k, k_stride, (const T*)v, v_stride, decay_pre,   \
-                     head_decay, bonus, state, state_stride, seg_start,         \
-                     seg_len, seg_slot, seg_fresh, H, D, Dv, TT, act_silu)
-#define LIG_MS(T, SP, KPT, B)                             \
-  do {                                                    \
-    if (threads <= 256) LIG_MS_T(T, SP, KPT, B, 256);     \
-    else LIG_MS_T(T, SP, KPT, B, 1024);                   \
-  } while (0)
-#define LIG_MS_K(T, B)                                    \
-  if (split == 8) {                                       \
-    switch (kpt) {                                        \
-      case 4: LIG_MS(T, 8, 4, B); break;                  \
-      case 8: LIG_MS(T, 8, 8, B); break;                  \
-      case 12: LIG_MS(T, 8, 12, B); break;                \
-      case 16: LIG_MS(T, 8, 16, B); break;                \
-      case 24: LIG_MS(T, 8, 24, B); break;                \
-      default: LIG_MS(T, 8, 32, B); break;                \
-    }                                                     \
-  } else {                                                \
-    switch (kpt) {                                        \
-      case 4: LIG_MS(T, 4, 4, B); break;                  \
-      case 8: LIG_MS(T, 4, 8, B); break;                  \
-      case 12: LIG_MS(T, 4, 12, B); break;                \
-      case 16: LIG_MS(T, 4, 16, B); break;                \
-      case 24: LIG_MS(T, 4, 24, B); break;                \
-      case 32: LIG_MS(T, 4, 32, B); break;                \
-      case 48: LIG_MS(T, 4, 48, B); break;                \
-      default: LIG_MS(T, 4, 64, B); break;                \
-    }                                                     \
-  }
+  const int threads = ((CBw * split + WAVE_SIZE - 1) / WAVE_SIZE) * WAVE_SIZE;
+  const MsArgs a{out, q, k, v, q_stride, k_stride, v_stride, decay_pre, head_decay, bonus,
+                 gate_i, gate_f, gate_stride, bias_i, bias_f, gate_cap, cs, nf, q_scale,
+                 k_scale, state, state_stride, seg_start, seg_len, seg_slot, seg_fresh,
+                 H, D, Dv, CB, NB, TT, act_silu};
+  const dim3 grid(S, H, NB);
+#define LIG_MS_FORM(T)                                                                        \
+  if (form == MS_BONUS) ms_dispatch<T, MS_BONUS>(a, split, kpt, grid, threads, smem, stream); \
+  else if (form == MS_GATED)                                                                  \
+    ms_dispatch<T, MS_GATED>(a, split, kpt, grid, threads, smem, stream);                     \
+  else ms_dispatch<T, MS_CONST>(a, split, kpt, grid, threads, smem, stream)
   if (is_f32) {
-    if (has_bonus) { LIG_MS_K(float, true) } else { LIG_MS_K(float, false) }
+    LIG_MS_FORM(float);
   } else {
-    if (has_bonus) { LIG_MS_K(bf16s, true) } else { LIG_MS_K(bf16s, false) }
+    LIG_MS_FORM(bf16s);
   }
-#undef LIG_MS_K
-#undef LIG_MS
-#undef LIG_MS_T
+#undef LIG_MS_FORM
   return 0;
 }

@@ -11,7 +11,8 @@
 //
 // group_rms_norm_gate: every `group` consecutive entries of an fp32 row are
 // divided by their root mean square (group == C: the whole row), times a
-// weight, times silu(gate) or sigmoid(gate).
+// weight (or none), times silu(gate) or sigmoid(gate); the result may be a
+// column block of a wider row.
 
 #include "elem_types.h"
 
@@ -88,14 +89,14 @@ __global__ __launch_bounds__(256) void scaled_add_rms_norm_vec_kernel(
 // group/4 neighbouring lanes and reduced with xor shuffles.
 template <typename T>
 __global__ __launch_bounds__(256) void group_rms_norm_gate_vec_kernel(
-    T* __restrict__ out, const float* __restrict__ o, const T* __restrict__ gate,
+    T* __restrict__ out, long out_stride, const float* __restrict__ o, const T* __restrict__ gate,
     long gate_stride, const T* __restrict__ w, int group, int gate_silu, float eps,
     int C) {
   __shared__ float red[17];
   const long r = blockIdx.x;
   const float* orow = o + r * C;
   const T* grow = gate + r * gate_stride;
-  T* out_row = out + r * C;
+  T* out_row = out + r * out_stride;
   const bool whole = group == C;
   float inv_whole = 0.f;
   if (whole) {
@@ -122,9 +123,9 @@ __global__ __launch_bounds__(256) void group_rms_norm_gate_vec_kernel(
       inv = 1.0f / sqrtf(ss / (float)group + eps);
     }
     if (live) {
-      float g[4], ww[4];
+      float g[4], ww[4] = {1.f, 1.f, 1.f, 1.f};
       ldn<4>(grow + c, g);
-      ldn<4>(w + c, ww);
+      if (w != nullptr) ldn<4>(w + c, ww);
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const float a = gate_silu ? g[i] * sigmoid_f32(g[i]) : sigmoid_f32(g[i]);
@@ -137,14 +138,14 @@ __global__ __launch_bounds__(256) void group_rms_norm_gate_vec_kernel(
 
 template <typename T>
 __global__ __launch_bounds__(256) void group_rms_norm_gate_kernel(
-    T* __restrict__ out, const float* __restrict__ o, const T* __restrict__ gate,
+    T* __restrict__ out, long out_stride, const float* __restrict__ o, const T* __restrict__ gate,
     long gate_stride, const T* __restrict__ w, int group, int gate_silu, float eps,
     int C) {
   __shared__ float red[17];
   const long r = blockIdx.x;
   const float* orow = o + r * C;
   const T* grow = gate + r * gate_stride;
-  T* out_row = out + r * C;
+  T* out_row = out + r * out_stride;
   if (group == C) {
     float ss = 0.f;
     for (int c = threadIdx.x; c < C; c += blockDim.x) {
@@ -156,7 +157,7 @@ __global__ __launch_bounds__(256) void group_rms_norm_gate_kernel(
     for (int c = threadIdx.x; c < C; c += blockDim.x) {
       const float g = ld(grow + c);
       const float a = gate_silu ? g * sigmoid_f32(g) : sigmoid_f32(g);
-      st(out_row + c, orow[c] * inv * ld(w + c) * a);
+      st(out_row + c, orow[c] * inv * (w ? ld(w + c) : 1.f) * a);
     }
     return;
   }
@@ -175,7 +176,7 @@ __global__ __launch_bounds__(256) void group_rms_norm_gate_kernel(
     for (int d = lane; d < group; d += WAVE_SIZE) {
       const float g = ld(grow + c0 + d);
       const float a = gate_silu ? g * sigmoid_f32(g) : sigmoid_f32(g);
-      st(out_row + c0 + d, orow[c0 + d] * inv * ld(w + c0 + d) * a);
+      st(out_row + c0 + d, orow[c0 + d] * inv * (w ? ld(w + c0 + d) : 1.f) * a);
     }
   }
 }
@@ -210,7 +211,7 @@ void lig_scaled_add_rms_norm(float* x, void* h, const void* y1, const void* y2,
                        (const bf16s*)w, alpha, s1, s2, eps, H);
 }
 
-void lig_group_rms_norm_gate(void* out, const float* o, const void* gate,
+void lig_group_rms_norm_gate(void* out, long out_stride, const float* o, const void* gate,
                              long gate_stride, const void* w, int group,
                              int gate_silu, float eps, int R, int C, int is_f32,
                              hipStream_t s) {
@@ -219,28 +220,28 @@ void lig_group_rms_norm_gate(void* out, const float* o, const void* gate,
   const int lanes = group / 4;
   const bool vec = C % 4 == 0 && group % 4 == 0 &&
                    (group == C || (lanes <= 64 && (lanes & (lanes - 1)) == 0)) &&
-                   aligned16(o) && gate_stride % 4 == 0 &&
+                   aligned16(o) && gate_stride % 4 == 0 && out_stride % 4 == 0 &&
                    (reinterpret_cast<uintptr_t>(gate) % (4 * esz)) == 0 &&
                    (reinterpret_cast<uintptr_t>(out) % (4 * esz)) == 0 &&
                    (reinterpret_cast<uintptr_t>(w) % (4 * esz)) == 0;
   if (vec) {
     if (is_f32)
       hipLaunchKernelGGL(group_rms_norm_gate_vec_kernel<float>, dim3(R), dim3(256), 0, s,
-                         (float*)out, o, (const float*)gate, gate_stride,
+                         (float*)out, out_stride, o, (const float*)gate, gate_stride,
                          (const float*)w, group, gate_silu, eps, C);
     else
       hipLaunchKernelGGL(group_rms_norm_gate_vec_kernel<bf16s>, dim3(R), dim3(256), 0, s,
-                         (bf16s*)out, o, (const bf16s*)gate, gate_stride,
+                         (bf16s*)out, out_stride, o, (const bf16s*)gate, gate_stride,
                          (const bf16s*)w, group, gate_silu, eps, C);
     return;
   }
   if (is_f32)
     hipLaunchKernelGGL(group_rms_norm_gate_kernel<float>, dim3(R), dim3(256), 0, s,
-                       (float*)out, o, (const float*)gate, gate_stride,
+                       (float*)out, out_stride, o, (const float*)gate, gate_stride,
                        (const float*)w, group, gate_silu, eps, C);
   else
     hipLaunchKernelGGL(group_rms_norm_gate_kernel<bf16s>, dim3(R), dim3(256), 0, s,
-                       (bf16s*)out, o, (const bf16s*)gate, gate_stride,
+                       (bf16s*)out, out_stride, o, (const bf16s*)gate, gate_stride,
                        (const bf16s*)w, group, gate_silu, eps, C);
 }
 

@@ -16,6 +16,11 @@
 // saw every token (ye = [experts, T, W]): row = idx * T + t, idx >= experts
 // being an identity expert.
 //
+// residual_routed_add: the same sum joined to the residual with the layer's
+// other branch in one pass, x += y + sum_k w[t, k] * ye[row[t, k]] (x fp32,
+// in place), and the new x rounded to T for the GEMM that reads it.  Without
+// ye only y is added.
+//
 // glu_act over a fused [gate | up] projection:
 //   0: relu(gate) * up
 //   1: g = min(gate, limit), u = clamp(up, -limit, limit),
@@ -42,14 +47,14 @@ LIG_DEVICE BestPair wave_argmax(BestPair b) {
 }
 
 __global__ __launch_bounds__(WAVE_SIZE) void grouped_topk_route_kernel(
-    const float* __restrict__ z, const float* __restrict__ corr, int N, int groups,
+    const float* __restrict__ z, long z_stride, const float* __restrict__ corr, int N, int groups,
     int keep, int top, int* __restrict__ idx_out, float* __restrict__ w_out) {
   extern __shared__ __align__(16) float sm[];
   float* s_s = sm;           // [N] scores
   float* c_s = sm + N;       // [N] choice scores, -inf once taken or barred
   float* g_s = sm + 2 * N;   // [groups]
   const int t = blockIdx.x, lane = threadIdx.x;
-  const float* zr = z + (long)t * N;
+  const float* zr = z + t * z_stride;
   float mx = -INFINITY;
   for (int i = lane; i < N; i += WAVE_SIZE) mx = fmaxf(mx, zr[i]);
   mx = wave_reduce_max(mx);
@@ -144,6 +149,33 @@ __global__ void routed_combine_kernel(T* __restrict__ out, const T* __restrict__
   }
 }
 
+template <typename T, int N>
+__global__ __launch_bounds__(256) void residual_routed_add_kernel(
+    float* __restrict__ x, T* __restrict__ xt, const T* __restrict__ y,
+    const T* __restrict__ ye, const long* __restrict__ rows, const int* __restrict__ idx,
+    const float* __restrict__ w, int top, int W) {
+  const long t = blockIdx.x;
+  const long ntok = gridDim.x;
+  for (int c = threadIdx.x * N; c < W; c += blockDim.x * N) {
+    float acc[N], v[N];
+    ldn<N>(y + t * W + c, acc);
+    if (ye != nullptr) {
+      for (int k = 0; k < top; ++k) {
+        const long r = rows != nullptr ? rows[t * top + k] : (long)idx[t * top + k] * ntok + t;
+        const float wk = w[t * top + k];
+        ldn<N>(ye + r * W + c, v);
+#pragma unroll
+        for (int i = 0; i < N; ++i) acc[i] += wk * v[i];
+      }
+    }
+    ldn<N>(x + t * W + c, v);
+#pragma unroll
+    for (int i = 0; i < N; ++i) v[i] += acc[i];
+    stn<N>(x + t * W + c, v);
+    if (xt != nullptr) stn<N>(xt + t * W + c, v);
+  }
+}
+
 template <typename T, int N, int KIND>
 __global__ void glu_act_kernel(T* __restrict__ out, const T* __restrict__ x, int F,
                                long n, float limit, float alpha) {
@@ -170,7 +202,7 @@ __global__ void glu_act_kernel(T* __restrict__ out, const T* __restrict__ x, int
 
 extern "C" {
 
-int lig_grouped_topk_route(const float* z, const float* corr, int T, int N,
+int lig_grouped_topk_route(const float* z, long z_stride, const float* corr, int T, int N,
                            int groups, int keep, int top, int* idx_out,
                            float* w_out, hipStream_t s) {
   if (N < 1 || top < 1 || top > N || groups < 1 || N % groups != 0 || keep < 1 ||
@@ -179,7 +211,7 @@ int lig_grouped_topk_route(const float* z, const float* corr, int T, int N,
   if (T <= 0) return 0;
   const size_t smem = (size_t)(2 * N + groups) * sizeof(float);
   hipLaunchKernelGGL(grouped_topk_route_kernel, dim3(T), dim3(WAVE_SIZE), smem, s, z,
-                     corr, N, groups, keep, top, idx_out, w_out);
+                     z_stride, corr, N, groups, keep, top, idx_out, w_out);
   return 0;
 }
 
@@ -198,6 +230,23 @@ void lig_routed_combine(void* out, const void* ye, const void* x, const long* ro
     if (v4) LIG_RC(bf16s, 4); else LIG_RC(bf16s, 1);
   }
 #undef LIG_RC
+}
+
+void lig_residual_routed_add(float* x, void* xt, const void* y, const void* ye,
+                             const long* rows, const int* idx, const float* w, int T,
+                             int top, int W, int is_f32, hipStream_t s) {
+  if (T <= 0 || W <= 0) return;
+  const bool v4 = W % 4 == 0 && aligned16(x) && aligned16(xt) && aligned16(y) && aligned16(ye);
+  const int threads = W >= 1024 ? 256 : (W >= 256 ? 128 : 64);
+#define LIG_RA(T_, N)                                                                      \
+  hipLaunchKernelGGL((residual_routed_add_kernel<T_, N>), dim3(T), dim3(threads), 0, s, x, \
+                     (T_*)xt, (const T_*)y, (const T_*)ye, rows, idx, w, top, W)
+  if (is_f32) {
+    if (v4) LIG_RA(float, 4); else LIG_RA(float, 1);
+  } else {
+    if (v4) LIG_RA(bf16s, 4); else LIG_RA(bf16s, 1);
+  }
+#undef LIG_RA
 }
 
 void lig_glu_act(void* out, const void* x, long rows, int F, int kind, float limit,

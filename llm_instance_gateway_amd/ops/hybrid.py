@@ -1,10 +1,11 @@
 """Light native library for the hybrid-model kernels (grouped RMS norm, xIELU,
 minGRU scan, general-size paged attention, shift norms, latent attention,
 sum+norm residual step, q/k/v prep, head-mixed attention, matrix-state scan,
-multi-stream residual step, grouped router and routed combine).
+multi-stream residual step, grouped router and routed combine, layer norms,
+fp32 projections onto a few columns).
 
 These kernels expose a plain C ABI and need no torch headers, so they are
-compiled by one direct ``hipcc -shared`` call (seconds, not the minutes the
+compiled by direct ``hipcc`` calls (side by side, without the minutes the
 torch extension takes) into ``llm_instance_gateway_amd/_hybrid.so`` and
 loaded with ctypes.  A model that needs only these kernels can therefore be
 served from a fresh checkout after a short first-use build; nothing else is
@@ -23,6 +24,7 @@ import os
 import shutil
 import subprocess
 import tempfile
+from concurrent.futures import ThreadPoolExecutor
 from pathlib import Path
 from typing import Optional
 
@@ -35,7 +37,7 @@ SOURCES = [
     "attention_prefill_tiles.hip", "shift_norm.hip", "latent_attention.hip", "ff_act.hip",
     "attention_latent_rows.hip", "post_norm.hip", "qkv_prep.hip", "attention_mixed_heads.hip",
     "matrix_state_scan.hip", "attention_mixed_heads_tiles.hip", "hyper_streams.hip",
-    "routed.hip",
+    "routed.hip", "layer_norm.hip", "small_projection.hip",
 ]
 SO_PATH = PKG / "_hybrid.so"
 
@@ -50,26 +52,34 @@ def _hipcc() -> str:
 
 
 def build() -> Path:
-    """Compile the light library for gfx950 (atomic replace of the .so)."""
-    fd, tmp = tempfile.mkstemp(prefix="._hybrid-", suffix=".so", dir=str(PKG))
-    os.close(fd)
-    cmd = [
-        _hipcc(), "-O3", "-std=c++17", "--offload-arch=gfx950",
-        "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
-        "-shared", "-fPIC", "-o", tmp,
-    ] + [str(CSRC / s) for s in SOURCES]
-    try:
-        subprocess.run(cmd, check=True, cwd=str(CSRC), stdout=subprocess.PIPE,
-                       stderr=subprocess.PIPE)
-        os.chmod(tmp, 0o755)
-        os.replace(tmp, SO_PATH)
-    except subprocess.CalledProcessError as e:
-        raise RuntimeError(
-            "building the hybrid kernel library failed:\n" + e.stderr.decode(errors="replace")[-4000:]
-        ) from None
-    finally:
-        if os.path.exists(tmp):
-            os.unlink(tmp)
+    """Compile the light library for gfx950: every source on its own, side by
+    side, then one link (atomic replace of the .so)."""
+    workers = max(1, min(8, len(os.sched_getaffinity(0)), int(os.environ.get("MAX_JOBS") or 8)))
+    flags = [
+        "-O3", "-std=c++17", "--offload-arch=gfx950",
+        "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-fPIC",
+    ]
+
+    def run(args) -> None:
+        try:
+            subprocess.run([_hipcc()] + flags + args, check=True, cwd=str(CSRC),
+                           stdout=subprocess.PIPE, stderr=subprocess.PIPE)
+        except subprocess.CalledProcessError as e:
+            raise RuntimeError(
+                "building the hybrid kernel library failed:\n"
+                + e.stderr.decode(errors="replace")[-4000:]
+            ) from None
+
+    with tempfile.TemporaryDirectory(prefix="._hybrid-", dir=str(PKG)) as tmp:
+        objs = [os.path.join(tmp, Path(s).stem + ".o") for s in SOURCES]
+        # the longest compilations first
+        jobs = sorted(zip(SOURCES, objs), key=lambda j: -(CSRC / j[0]).stat().st_size)
+        with ThreadPoolExecutor(max_workers=workers) as pool:
+            list(pool.map(lambda j: run(["-c", str(CSRC / j[0]), "-o", j[1]]), jobs))
+        so = os.path.join(tmp, "_hybrid.so")
+        run(["-shared", "-o", so] + objs)
+        os.chmod(so, 0o755)
+        os.replace(so, SO_PATH)
     return SO_PATH
 
 
@@ -90,9 +100,12 @@ def _declare(lib: ctypes.CDLL) -> None:
         "lig_offset_rms_norm": [p, p, p, f, i, i, i, p],
         "lig_residual_add": [p, p, p, l, i, p],
         "lig_latent_kv_prep": [p, p, l, p, p, p, i, p, p, p, f, i, i, i, i, i, p],
-        "lig_rotate_pack_queries": [p, p, p, i, p, i, i, i, i, i, i, p],
+        "lig_rotate_pack_queries": [p, p, l, p, i, p, i, i, i, i, i, i, p],
+        "lig_rotary_table": [p, p, p, i, i, p],
         "lig_scale_gather_rows": [p, p, p, p, l, i, i, p],
         "lig_relu_squared": [p, p, l, i, p],
+        "lig_relu_squared_rows": [p, l, p, l, l, i, i, p],
+        "lig_gelu_tanh_table_mul": [p, p, p, l, p, l, i, i, p],
         "lig_silu_mul": [p, p, l, i, i, p],
         "lig_kv_scatter": [p, p, l, p, p, p, i, i, i, i, i, i, p],
         "lig_temperature_scale_rows": [p, p, l, p, f, f, i, i, i, i, p],
@@ -101,12 +114,13 @@ def _declare(lib: ctypes.CDLL) -> None:
             p, p, p, l, p, p, p, i, p, p, f, p, p, p, f, i, i, i, i, i, i, i, i, i, i, i, p,
         ],
         "lig_token_shift_mix": [p, p, p, p, p, p, p, p, p, i, i, i, i, p],
-        "lig_group_rms_norm_gate": [p, p, p, l, p, i, i, f, i, i, i, p],
+        "lig_group_rms_norm_gate": [p, l, p, p, l, p, i, i, f, i, i, i, p],
         "lig_gelu_erf": [p, p, l, i, p],
         "lig_tanh_act": [p, p, l, i, p],
         "lig_tanh_softcap": [p, f, l, p],
         "lig_routed_combine": [p, p, p, p, p, i, p, i, i, i, i, p],
         "lig_glu_act": [p, p, l, i, i, f, f, i, p],
+        "lig_residual_routed_add": [p, p, p, p, p, p, p, i, i, i, i, p],
     }
     for name, args in sigs.items():
         fn = getattr(lib, name)
@@ -122,8 +136,14 @@ def _declare(lib: ctypes.CDLL) -> None:
     hs.argtypes = [p, p, p, p, f, p, p, f, p, i, i, i, i, p]
     hs.restype = ctypes.c_int
     gr = lib.lig_grouped_topk_route
-    gr.argtypes = [p, p, i, i, i, i, i, p, p, p]
+    gr.argtypes = [p, l, p, i, i, i, i, i, p, p, p]
     gr.restype = ctypes.c_int
+    sp = lib.lig_small_projection
+    sp.argtypes = [p, p, p, i, i, i, p]
+    sp.restype = ctypes.c_int
+    ln = lib.lig_layer_norm
+    ln.argtypes = [p, p, p, p, f, p, p, p, f, i, i, i, p]
+    ln.restype = ctypes.c_int
     mh = lib.lig_paged_attention_mixed_heads
     mh.argtypes = [p, p, l, p, p, p, i, p, p, p, i, p, f, i, i, i, i, i, i, i, i, p]
     mh.restype = ctypes.c_int
@@ -131,10 +151,13 @@ def _declare(lib: ctypes.CDLL) -> None:
     mt.argtypes = [p, p, l, p, p, p, i, p, p, p, p, p, p, f, i, i, i, i, i, i, i, i, p]
     mt.restype = ctypes.c_int
     ms = lib.lig_matrix_state_scan
-    ms.argtypes = [p, p, l, p, l, p, l, p, p, p, p, l, p, p, p, p, i, i, i, i, i, i, p]
+    ms.argtypes = [
+        p, p, l, p, l, p, l, p, p, p, p, p, l, p, p, f, p, i, f, f, p, l, p, p, p, p,
+        i, i, i, i, i, i, p,
+    ]
     ms.restype = ctypes.c_int
     lr = lib.lig_latent_attention_rows
-    lr.argtypes = [p, p, p, p, p, p, p, p, i, f, i, i, i, i, i, i, i, p, p]
+    lr.argtypes = [p, p, p, p, p, l, p, p, p, p, i, f, i, i, i, i, i, i, i, p, p]
     lr.restype = ctypes.c_int
 
 

@@ -444,7 +444,7 @@ def latent_kv_prep(
     latent followed by the rotated key part into cache row slot_mapping[r]
     (cache [blocks, 1, block_size, kv_rank + rot_dim])."""
     a, b = q_rank, q_rank + kv_rank
-    cq = (_rms_scale(proj[:, :a], eps) * w_q.float()).to(proj.dtype)
+    cq = proj[:, :0] if w_q is None else (_rms_scale(proj[:, :a], eps) * w_q.float()).to(proj.dtype)
     c = _rms_scale(proj[:, a:b], eps) * w_kv.float()
     kr = _rotate_pairs(proj[:, b : b + rot_dim], positions, inv_freq)
     row = torch.cat([c, kr], dim=-1).to(cache.dtype)
@@ -458,9 +458,19 @@ def rotate_pack_queries(q, heads: int, dim: int, rot_dim: int, inv_freq, positio
     """out[r, h, lead:lead+rot_dim] = rotated q[r, h, dim:dim+rot_dim]; q is
     [R, heads*(dim+rot_dim)], out [R, heads, lead+rot_dim]."""
     R = q.shape[0]
-    qr = q.view(R, heads, dim + rot_dim)[:, :, dim:]
+    qr = q.unflatten(1, (heads, dim + rot_dim))[:, :, dim:]
     out[:, :, lead:] = _rotate_pairs(qr, positions, inv_freq).to(out.dtype)
     return out
+
+
+def rotary_table(positions: torch.Tensor, inv_freq: torch.Tensor) -> torch.Tensor:
+    ang = positions.float()[:, None] * inv_freq[None, :]
+    return torch.cat([torch.cos(ang), torch.sin(ang)], dim=1)
+
+
+def gelu_tanh_table_mul(z, table, tokens) -> torch.Tensor:
+    g = torch.nn.functional.gelu(z.float(), approximate="tanh")
+    return (g * table[tokens].float()).to(z.dtype)
 
 
 def relu_squared(x: torch.Tensor) -> torch.Tensor:
@@ -602,16 +612,28 @@ def token_shift_mix(x, mu, state, seg_start, seg_len, seg_slot, seg_fresh, out_d
 def matrix_state_scan(
     q, k, v, state, seg_start, seg_len, seg_slot, seg_fresh, heads: int, dim: int,
     vdim: int, decay_pre=None, head_decay=None, bonus=None, act_silu: bool = False,
+    gates=None, gate_bias=None, gate_cap: float = 1.0, rot=None, q_scale: float = 1.0,
+    k_scale: float = 1.0,
 ):
     """Per head a [dim, vdim] fp32 state S.  With `bonus` u (per head and key
     channel): o_t = (S + diag(u) k_t v_t^T)^T q_t, then S <- diag(w_t) S +
     k_t v_t^T with w_t = exp(-exp(decay_pre_t)).  Without: S <- d_h S + k_t
-    v_t^T with the head's constant d_h, then o_t = S^T q_t.  act_silu applies
-    silu to q, k and v first.  State rows [slots, heads*dim*vdim] are read
-    unless the segment starts its sequence, and written back."""
+    v_t^T with the head's constant d_h, then o_t = S^T q_t.  With gates: the
+    stabilised input / forget gates with a normaliser vector n (its state
+    beside the matrix, then the running maximum).  act_silu applies silu to
+    q, k and v first, then q and k are rotated (`rot`) and scaled.  State
+    rows are read unless the segment starts its sequence, and written back."""
     R = q.shape[0]
     f = (lambda t: torch.nn.functional.silu(t.float())) if act_silu else (lambda t: t.float())
     qf, kf, vf = f(q).view(R, heads, dim), f(k).view(R, heads, dim), f(v).view(R, heads, vdim)
+    if rot is not None:
+        qf, kf = _rotate_halves_table(qf, rot), _rotate_halves_table(kf, rot)
+    qf, kf = qf * q_scale, kf * k_scale
+    if gates is not None:
+        return _gated_matrix_state_scan(
+            qf, kf, vf, state, seg_start, seg_len, seg_slot, seg_fresh,
+            *(gate_cap * torch.tanh((g.float() + b.float()) / gate_cap) for g, b in zip(gates, gate_bias)),
+        )
     out = torch.zeros(R, heads, vdim, dtype=torch.float32, device=q.device)
     w = None
     if decay_pre is not None:
@@ -637,11 +659,50 @@ def matrix_state_scan(
     return out.view(R, heads * vdim)
 
 
+def _rotate_halves_table(v: torch.Tensor, cs: torch.Tensor) -> torch.Tensor:
+    """v [R, H, D] fp32: entries i and i + n of every head turn by the angle
+    whose cosine and sine are cs[r, i] and cs[r, n + i]."""
+    n = cs.shape[1] // 2
+    c, s = cs[:, None, :n], cs[:, None, n:]
+    a, b = v[..., :n], v[..., n : 2 * n]
+    return torch.cat([a * c - b * s, b * c + a * s, v[..., 2 * n :]], dim=-1)
+
+
+def _gated_matrix_state_scan(q, k, v, state, seg_start, seg_len, seg_slot, seg_fresh, gi, gf):
+    R, H, D = q.shape
+    Dv = v.shape[-1]
+    gf = torch.nn.functional.logsigmoid(gf)
+    v1 = torch.cat([v, torch.ones(R, H, 1, dtype=v.dtype, device=v.device)], dim=-1)
+    out = torch.zeros(R, H, Dv, dtype=torch.float32, device=q.device)
+    nS = H * D * (Dv + 1)
+    for s0, n, slot, fresh in zip(
+        seg_start.tolist(), seg_len.tolist(), seg_slot.tolist(), seg_fresh.tolist()
+    ):
+        if n <= 0:
+            continue
+        S = torch.zeros(H, D, Dv + 1, device=q.device)  # the last column is the normaliser
+        m = torch.zeros(H, device=q.device)
+        if not fresh:
+            S, m = state[slot, :nS].view(H, D, Dv + 1).clone(), state[slot, nS : nS + H].clone()
+        for t in range(s0, s0 + n):
+            m_new = torch.maximum(gf[t] + m, gi[t])
+            a, b = torch.exp(gf[t] + m - m_new), torch.exp(gi[t] - m_new)
+            m = m_new
+            S = a[:, None, None] * S + (b[:, None] * k[t])[:, :, None] * v1[t][:, None, :]
+            o = torch.einsum("hd,hde->he", q[t], S)
+            out[t] = o[:, :Dv] / (torch.maximum(o[:, Dv].abs(), torch.exp(-m)) + 1e-6)[:, None]
+        state[slot, :nS] = S.reshape(-1)
+        state[slot, nS : nS + H] = m
+    return out.view(R, H * Dv)
+
+
 def group_rms_norm_gate(o, gate, w, group: int, gate_act: str, eps: float, out_dtype):
     """Every `group` consecutive entries of a row are divided by their root
     mean square; then times w, times silu(gate) or sigmoid(gate)."""
     R, C = o.shape
-    n = _rms_scale(o.view(R, C // group, group), eps).view(R, C) * w.float()
+    n = _rms_scale(o.view(R, C // group, group), eps).view(R, C)
+    if w is not None:
+        n = n * w.float()
     g = gate.float()
     g = torch.nn.functional.silu(g) if gate_act == "silu" else torch.sigmoid(g)
     return (n * g).to(out_dtype)
@@ -693,6 +754,27 @@ def routed_combine(ye, x, rows, w):
     src = torch.cat([ye, x], dim=0).float()
     at = torch.where(rows >= 0, rows, ye.shape[0] + torch.arange(T, device=x.device)[:, None])
     return (src[at] * w[:, :, None]).sum(dim=1).to(x.dtype)
+
+
+def residual_routed_add(x, y, ye, w, rows):
+    x.add_(y.float() if ye is None else y.float() + (ye.float()[rows] * w[:, :, None]).sum(dim=1))
+    return x.to(y.dtype)
+
+
+def layer_norm(x, w, eps: float) -> torch.Tensor:
+    d = x.float() - x.float().mean(dim=-1, keepdim=True)
+    return (d * torch.rsqrt(d.pow(2).mean(dim=-1, keepdim=True) + eps) * w.float()).to(w.dtype)
+
+
+def embed_layer_norm(tokens, table, scale: float, w, eps: float):
+    x = table[tokens].float() * scale
+    return x, layer_norm(x, w, eps)
+
+
+def add_layer_norm(x, w, eps: float, y=None, w_y=None):
+    if y is not None:
+        x.add_(_rms_scale(y, eps) * w_y.float())
+    return layer_norm(x, w, eps)
 
 
 def glu_act(x, kind: str, limit: float, alpha: float):
