@@ -1,0 +1,461 @@
+"""The ops behind the Garesun blocks, each alone, against the float64 oracle in
+garesun_oracle.py.  CPU parametrisation: the torch execution path; `gpu`: the
+HIP kernels in fp32 and bf16 storage.
+
+Where random inputs would hide a fault they are constructed: one key scaled
+until its score stands out (far back, at page borders, at the query itself and
+one past it), one token of a recurrence that dominates everything after it,
+gates that saturate, stale content in reused slots and cache rows.
+"""
+
+import math
+
+import pytest
+import torch
+
+from llm_instance_gateway_amd import ops
+from llm_instance_gateway_amd.models.hybrid_blocks import (
+    LatentAttention, ReluSquaredExpertsMLP, ScalarDecayMixer, TokenTableGate,
+)
+
+import garesun_oracle as O
+
+F64 = torch.float64
+CASES = [("cpu", torch.float32), pytest.param("cuda:0", torch.float32, marks=pytest.mark.gpu),
+         pytest.param("cuda:0", torch.bfloat16, marks=pytest.mark.gpu)]
+
+
+def rnd(g, *shape, s=1.0):
+    return torch.randn(*shape, generator=g) * s
+
+
+def close(got, want, dtype, scale=None, tol32=2e-5):
+    want = want.to(F64)
+    ref = max(want.abs().max().item(), 1e-30) if scale is None else scale
+    err = (got.detach().double().cpu() - want).abs().max().item() / ref
+    assert err < (tol32 if dtype == torch.float32 else 2e-2), err
+
+
+def i32(v, dev):
+    return torch.tensor(v, dtype=torch.int32, device=dev)
+
+
+# -- norms ------------------------------------------------------------------------
+
+@pytest.mark.parametrize("device,dtype", CASES)
+@pytest.mark.parametrize("H", [7, 36, 50, 1028, 4100])
+def test_layer_norms(device, dtype, H):
+    """A large common offset: the deviations are what is normed."""
+    g = torch.Generator().manual_seed(H)
+    R, V, eps = 5, 11, 1e-3
+    table, w, wy = rnd(g, V, H).to(dtype), (1 + 0.3 * rnd(g, H)).to(dtype), (1 + 0.3 * rnd(g, H)).to(dtype)
+    toks = torch.tensor([3, 0, 10, 3, 7])
+    x, h = ops.embed_layer_norm(toks.to(device), table.to(device), 7.5, w.to(device), eps)
+    want = table[toks].to(F64) * 7.5
+    assert x.dtype == torch.float32 and h.dtype == dtype
+    close(x, want, torch.float32, tol32=1e-6)
+    close(h, O.layer_norm(want, w.to(F64), eps), dtype)
+
+    x0, y = rnd(g, R, H, s=2) + 30.0, rnd(g, R, H, s=5).to(dtype)
+    xs = x0.clone().to(device)
+    close(ops.add_layer_norm(xs, w.to(device), eps), O.layer_norm(x0.to(F64), w.to(F64), eps), dtype, tol32=2e-4)
+    assert torch.equal(xs.cpu(), x0)
+    want_x = x0.to(F64) + O.unit_rms(y.to(F64), eps) * wy.to(F64)
+    h = ops.add_layer_norm(xs, w.to(device), eps, y.to(device), wy.to(device))
+    close(xs, want_x, torch.float32, tol32=1e-6)
+    close(h, O.layer_norm(want_x, w.to(F64), eps), dtype, tol32=2e-4)
+
+
+# -- projections, activations, residual ---------------------------------------------
+
+@pytest.mark.parametrize("device,dtype", CASES)
+@pytest.mark.parametrize("R,N,C", [(1, 3, 40), (17, 16, 264), (33, 40, 96), (5, 70, 520), (6, 9, 50)])
+def test_small_projection_is_fp32(device, dtype, R, N, C):
+    g = torch.Generator().manual_seed(N)
+    h, w = rnd(g, R, C).to(dtype), rnd(g, N, C).to(dtype)
+    got = ops.small_projection(h.to(device), w.to(device))
+    assert got.dtype == torch.float32
+    close(got, h.to(F64) @ w.to(F64).T, torch.float32)  # fp32 sums in both storage types
+
+
+@pytest.mark.parametrize("device,dtype", CASES)
+def test_activations_between_column_blocks(device, dtype):
+    g = torch.Generator().manual_seed(2)
+    for R, F in ((6, 12), (5, 7)):
+        wide, out = rnd(g, R, F + 8).to(dtype).to(device), torch.full((R, F + 4), 9.0, dtype=dtype, device=device)
+        ops.relu_squared(wide[:, 8:], out=out[:, 4:])
+        close(out[:, 4:], torch.relu(wide[:, 8:].cpu().to(F64)) ** 2, dtype)
+        assert (out[:, :4] == 9.0).all()
+        table, toks = rnd(g, 9, 3 * F).to(dtype).to(device), torch.randint(0, 9, (R,), generator=g)
+        z = rnd(g, R, F, s=2).to(dtype).to(device)
+        got = ops.gelu_tanh_table_mul(z, table[:, F : 2 * F], toks.to(device))
+        close(got, O.gelu_tanh(z.cpu().to(F64)) * table.cpu().to(F64)[toks, F : 2 * F], dtype)
+    gate = TokenTableGate(24, 5, device, dtype)
+    with torch.no_grad():
+        gate.w_gate.copy_(rnd(g, 5, 24)); gate.w_proj.copy_(rnd(g, 24, 5)); gate.norm.copy_(1 + 0.2 * rnd(g, 24))
+    x, table, toks = rnd(g, 6, 24).to(dtype), rnd(g, 8, 15).to(dtype), torch.tensor([1, 7, 0, 1, 3, 2])
+    W = {"l2.side.gate": gate.w_gate.cpu().to(F64), "l2.side.proj": gate.w_proj.cpu().to(F64),
+         "l2.side.norm": gate.norm.cpu().to(F64), "side.embed": table.to(F64)}
+    y = gate(x.to(device), table.to(device)[:, 10:15], toks.to(device))
+    got = O.unit_rms(y.cpu().to(F64), 1e-5) * W["l2.side.norm"]
+    close(got, O.token_side(x.to(F64), toks, W, 2, 5, 1e-5), dtype, tol32=1e-4)
+
+
+@pytest.mark.parametrize("device,dtype", CASES)
+@pytest.mark.parametrize("W_", [12, 13])
+def test_residual_routed_add(device, dtype, W_):
+    g = torch.Generator().manual_seed(3)
+    R, E, top, cap = 6, 4, 3, 5
+    x, y = rnd(g, R, W_, s=4), rnd(g, R, W_).to(dtype)
+    ye, w = rnd(g, E * cap, W_).to(dtype), torch.rand(R, top, generator=g)
+    rows = torch.randint(0, E * cap, (R, top), generator=g)
+    want = x.to(F64) + y.to(F64) + (ye.to(F64)[rows] * w.to(F64)[:, :, None]).sum(1)
+    xs = x.clone().to(device)
+    xt = ops.residual_routed_add(xs, y.to(device), ye.to(device), w.to(device), rows.to(device))
+    close(xs, want, torch.float32, tol32=1e-6)
+    close(xt, want, dtype, tol32=1e-6)
+    assert xt.dtype == dtype
+    # every expert saw every token: rows follow from the choices
+    ye = rnd(g, E * R, W_).to(dtype)
+    idx = torch.stack([torch.randperm(E, generator=g)[:top] for _ in range(R)]).to(torch.int32)
+    want = x.to(F64) + y.to(F64)
+    for t in range(R):
+        for k in range(top):
+            want[t] += w[t, k].to(F64) * ye[int(idx[t, k]) * R + t].to(F64)
+    xs = x.clone().to(device)
+    ops.residual_routed_add(xs, y.to(device), ye.to(device), w.to(device), idx=idx.to(device), experts=E)
+    close(xs, want, torch.float32, tol32=1e-6)
+    xs = x.clone().to(device)
+    ops.residual_routed_add(xs, y.to(device))
+    close(xs, x.to(F64) + y.to(F64), torch.float32, tol32=1e-6)
+
+
+# -- routed experts -------------------------------------------------------------------
+
+@pytest.mark.parametrize("device", ["cpu", pytest.param("cuda:0", marks=pytest.mark.gpu)])
+@pytest.mark.parametrize("N,top", [(8, 3), (1, 1), (5, 5), (70, 2)])
+def test_router_is_a_softmax_over_the_chosen(device, N, top):
+    g = torch.Generator().manual_seed(N)
+    wide = rnd(g, 9, N + 6, s=3)
+    wide[0, :N] = torch.arange(N) * (60.0 / N)  # one choice far above the rest
+    idx, w = ops.grouped_topk_route(wide.to(device)[:, :N], None, top)
+    for t in range(9):
+        ref_i, ref_w = O.route(wide[t, :N].to(F64), top)
+        assert idx[t].tolist() == ref_i
+        close(w[t], torch.tensor(ref_w), torch.float32, scale=1.0, tol32=1e-6)
+
+
+class _Meta:
+    def __init__(self, np_):
+        self.num_prefill_tokens = np_
+
+
+@pytest.mark.parametrize("device,dtype", CASES)
+@pytest.mark.parametrize("E,top,shared", [(6, 2, 20), (1, 1, 0), (3, 3, 8), (5, 1, 16)])
+def test_squared_relu_experts_both_dispatch_paths(device, dtype, E, top, shared):
+    g = torch.Generator().manual_seed(E)
+    H, ff, T = 24, 16, 11
+    mlp = ReluSquaredExpertsMLP(H, ff, E, top, shared, device=device, dtype=dtype)
+    W = {"router": rnd(g, E, H)}
+    for e in range(E):
+        W[f"e{e}.up"], W[f"e{e}.down"] = rnd(g, ff, H, s=0.3), rnd(g, H, ff, s=0.3)
+    if shared:
+        W["shared.up"], W["shared.down"] = rnd(g, shared, H, s=0.3), rnd(g, H, shared, s=0.3)
+    W = {k: v.to(dtype) for k, v in W.items()}
+    mlp.load(lambda n: W[n].to(device), "")
+    h = rnd(g, T, H).to(dtype)
+    cfg = {"router": {"top": top}, "shared": {"ff": shared} if shared else None}
+    want = O.moe_ff(h.to(F64), {k: v.to(F64) for k, v in W.items()}, "", cfg)
+    for meta in (_Meta(4), _Meta(0)):  # gathered batches, then every expert on every token
+        close(mlp(h.to(device), meta), want, dtype)
+
+
+# -- matrix-state recurrences ------------------------------------------------------------
+
+def scan_in_cuts(device, data, plans, slots, heads, dim, vdim, gated, make_kw):
+    """Feed several sequences portion by portion through one state pool full of
+    junk; returns {sequence: rows}.  `make_kw(index rows)` gives the op's
+    per-token arguments for the flat batch."""
+    width = ops.matrix_state_width(heads, dim, vdim, gated)
+    state = torch.full((max(slots.values()) + 2, width), 5.0, device=device)
+    at = {s: 0 for s in data}
+    got = {s: [] for s in data}
+    for plan in plans:
+        start, ln, sl, fresh, rows = [], [], [], [], []
+        for s, n in plan:
+            start.append(sum(ln)); ln.append(n); sl.append(slots[s]); fresh.append(int(at[s] == 0))
+            rows += [(s, t) for t in range(at[s], at[s] + n)]
+            at[s] += n
+        fused = torch.stack([data[s][t] for s, t in rows]).to(device)
+        a, b = heads * dim, 2 * heads * dim
+        o = ops.matrix_state_scan(
+            fused[:, :a], fused[:, a:b], fused[:, b : b + heads * vdim], state, i32(start, device),
+            i32(ln, device), i32(sl, device), i32(fresh, device), heads, dim, vdim, **make_kw(rows),
+        )
+        assert o.dtype == torch.float32
+        for (s, n), r0 in zip(plan, start):
+            got[s].append(o[r0 : r0 + n].cpu())
+    return {s: torch.cat(v) for s, v in got.items()}
+
+
+def plans_for(cuts, other):
+    """Sequence 0 in `cuts`; sequence 1 joins with portions of two tokens."""
+    out = []
+    for i, n in enumerate(cuts):
+        out.append([(0, n)] + ([(1, 2)] if i * 2 < other else []))
+    return out
+
+
+CUTS = [[147], [20, 2, 1, 64, 60], [2] * 10 + [127], [1] * 60 + [87], [64, 64, 19], [130, 17]]
+
+
+@pytest.mark.parametrize("device,dtype", CASES)
+@pytest.mark.parametrize("heads,dim,vdim,rot", [(3, 10, 6, 4), (2, 32, 64, 32), (1, 40, 65, 16), (2, 8, 130, 0),
+                                                (2, 64, 128, 64), (1, 128, 40, 128), (4, 16, 16, 16)])
+def test_retention_scan(device, dtype, heads, dim, vdim, rot):
+    """Rotated q and k, scaled k, one decay per head (also exactly 1)."""
+    g = torch.Generator().manual_seed(dim)
+    base, T = 300.0, {0: 147, 1: 12}
+    decay = [0.5, 0.99, 1.0, 0.9995][:heads] if heads > 1 else [0.97]
+    nq = heads * dim
+    data, want, pos0 = {}, {}, {0: 900, 1: 0}
+    for s, n in T.items():
+        x = torch.cat([rnd(g, n, nq), rnd(g, n, nq), rnd(g, n, heads * vdim)], dim=1)
+        if s == 0:
+            x[3, nq:] *= 8.0  # one early token dominates what follows
+        data[s] = x.to(dtype)
+        xd = data[s].to(F64)
+        q, k, v = (t.view(n, heads, -1) for t in (xd[:, :nq], xd[:, nq : 2 * nq], xd[:, 2 * nq :]))
+        pos = torch.arange(n) + pos0[s]
+        if rot:
+            q, k = O.rotate_halves(q, pos, base, rot), O.rotate_halves(k, pos, base, rot)
+        want[s] = O.retention_recurrence(q, k * dim ** -0.5, v, decay)[0].reshape(n, -1)
+    hd = torch.tensor(decay, device=device)
+    freq = ops.rotary_inv_freq(base, rot, device) if rot else None
+
+    def kw(rows):
+        pos = torch.tensor([pos0[s] + t for s, t in rows], device=device)
+        return dict(head_decay=hd, k_scale=dim ** -0.5, rot=ops.rotary_table(pos, freq) if rot else None)
+
+    for cuts in CUTS:
+        got = scan_in_cuts(device, data, plans_for(cuts, 2 * min(len(cuts), 6)), {0: 2, 1: 0}, heads, dim, vdim, False, kw)
+        for s in got:
+            # rotated angles at position ~1000 carry 1e-4 of fp32 rounding
+            close(got[s], want[s][: got[s].shape[0]], torch.float32, scale=want[s].abs().max().item(), tol32=2e-4)
+
+
+def gate_case(kind, g, n, heads):
+    """(input gate logits, forget gate logits) [n, heads]."""
+    i, f = rnd(g, n, heads, s=2), rnd(g, n, heads, s=2) + 2
+    if kind == "forget":      # forget gates near zero now and then: the state restarts
+        f[::9] = -30.0
+    elif kind == "spike":     # one input gate far above everything after it
+        i[5] = 25.0
+    elif kind == "keep":      # nothing is forgotten, tiny inputs: exp(-m) rules the denominator
+        i, f = i - 9.0, f + 20.0
+    elif kind == "late":      # m follows the forget gates down, then jumps
+        i[: n // 2] = -30.0
+        f[: n // 2] = -6.0
+    return i, f
+
+
+@pytest.mark.parametrize("device,dtype", CASES)
+@pytest.mark.parametrize("kind", ["plain", "forget", "spike", "keep", "late"])
+@pytest.mark.parametrize("heads,dim,vdim", [(2, 24, 40), (1, 48, 64), (3, 9, 5), (1, 33, 130), (2, 128, 64)])
+def test_mlstm_scan(device, dtype, kind, heads, dim, vdim):
+    g = torch.Generator().manual_seed(heads * 100 + dim)
+    cap, T, nq = 9.0, {0: 147, 1: 12}, heads * dim
+    b_i, b_f = rnd(g, heads), rnd(g, heads)
+    data, gates, want = {}, {}, {}
+    for s, n in T.items():
+        data[s] = torch.cat([rnd(g, n, nq), rnd(g, n, nq), rnd(g, n, heads * vdim)], dim=1).to(dtype)
+        gi, gf = gate_case(kind, g, n, heads)
+        gates[s] = torch.cat([gi, gf], dim=1)
+        xd = data[s].to(F64)
+        q, k, v = (t.view(n, heads, -1) for t in (xd[:, :nq], xd[:, nq : 2 * nq], xd[:, 2 * nq :]))
+        ident = {"i": torch.eye(heads, dtype=F64), "f": torch.eye(heads, dtype=F64), "i.b": b_i.to(F64), "f.b": b_f.to(F64)}
+        i, _ = O.mlstm_gates(gi.to(F64), ident, "", cap)
+        _, f = O.mlstm_gates(gf.to(F64), ident, "", cap)
+        want[s] = O.mlstm_recurrence(q * dim ** -0.5, k, v, i, f)[0].reshape(n, -1)
+
+    def kw(rows):
+        z = torch.stack([torch.cat([torch.zeros(3), gates[s][t]]) for s, t in rows]).to(device)
+        return dict(gates=(z[:, 3 : 3 + heads], z[:, 3 + heads :]), gate_bias=(b_i.to(device), b_f.to(device)),
+                    gate_cap=cap, q_scale=dim ** -0.5)
+
+    for cuts in CUTS:
+        got = scan_in_cuts(device, data, plans_for(cuts, 2 * min(len(cuts), 6)), {0: 2, 1: 0}, heads, dim, vdim, True, kw)
+        for s in got:
+            w = want[s][: got[s].shape[0]]
+            # a denominator |n . q| near zero magnifies rounding: row-wise scale
+            scale = w.abs().amax(dim=1, keepdim=True).clamp(min=w.abs().mean().item())
+            e = ((got[s].double() - w) / scale).abs().amax(dim=1)
+            assert e.max().item() < 2e-3 and e.median().item() < 2e-5, (kind, cuts, e.max().item(), e.median().item())
+
+
+@pytest.mark.parametrize("device,dtype", CASES)
+def test_mlstm_maximum_starts_at_zero(device, dtype):
+    """First token with a small input gate: m = max(f + 0, i) = f, and exp(-m)
+    bounds the denominator from below; a start at minus infinity would give
+    m = i and another output."""
+    data = {0: torch.tensor([[0.5, 0.25, 2.0]]).to(dtype)}
+    z = torch.tensor([[-4.0, 3.0]], device=device)
+
+    def kw(rows):
+        zero = torch.zeros(1, device=device)
+        return dict(gates=(z[:, :1], z[:, 1:]), gate_bias=(zero, zero), gate_cap=100.0)
+
+    got = scan_in_cuts(device, data, [[(0, 1)]], {0: 0}, 1, 1, 1, True, kw)[0]
+    i, f = 100 * math.tanh(-0.04), O.log_sigmoid(100 * math.tanh(0.03))
+    m = max(f, i)
+    b = math.exp(i - m)
+    want = b * 0.25 * 2.0 * 0.5 / (max(abs(b * 0.25 * 0.5), math.exp(-m)) + 1e-6)
+    close(got, torch.tensor([[want]], dtype=F64), torch.float32, tol32=1e-5)
+
+
+@pytest.mark.parametrize("device,dtype", CASES)
+@pytest.mark.parametrize("kind", ["retention", "mlstm"])
+def test_scalar_decay_mixer_whole(device, dtype, kind):
+    g = torch.Generator().manual_seed(11)
+    hidden, heads, dim, vdim, T, eps = 40, 3, 12, 20, 37, 1e-4
+    m = {"heads": heads, "dim": dim, "vdim": vdim, "decay": [0.6, 0.95, 0.999], "gate_cap": 5.0,
+         "rot": {"base": 50.0, "dims": 8}}
+    mix = ScalarDecayMixer(hidden, kind, heads, dim, vdim, eps, decay=m["decay"], rot_base=50.0,
+                           rot_dims=8 if kind == "retention" else 0, gate_cap=5.0, device=device, dtype=dtype)
+    W = {n: rnd(g, r, hidden, s=hidden ** -0.5).to(dtype) for n, r in
+         (("q", heads * dim), ("k", heads * dim), ("v", heads * vdim), ("g", heads * vdim), ("i", heads), ("f", heads))}
+    W["o"] = rnd(g, hidden, heads * vdim, s=0.2).to(dtype)
+    W["norm"], W["i.b"], W["f.b"] = (1 + 0.2 * rnd(g, heads * vdim)).to(dtype), rnd(g, heads).to(dtype), (rnd(g, heads) + 2).to(dtype)
+    mix.load(lambda n: W[n].to(device), "")
+    h = rnd(g, T, hidden).to(dtype)
+    Wd = {k: v.to(F64) for k, v in W.items()}
+    want = (O.retention if kind == "retention" else O.mlstm)(h.to(F64), Wd, "", m, eps)
+
+    class Meta:
+        seg_start, seg_len, seg_slot, seg_fresh = i32([0], device), i32([T], device), i32([1], device), i32([1], device)
+        num_prefill_tokens, num_decode_tokens = T, 0
+
+    state = torch.full((3, mix.cache_spec()["width"]), 7.0, device=device)
+    got = mix(h.to(device), torch.arange(T, device=device), (state,), Meta)
+    close(got, want, dtype, tol32=2e-4)
+
+
+# -- latent attention with direct queries, a gate per head and shared rows ------------------
+
+def latent_batch(device, bs, lens, ctx, pages):
+    """Segments of `lens` new tokens that end at contexts `ctx`, over scattered pages."""
+    g = torch.Generator().manual_seed(5)
+    nblk = [(c + bs - 1) // bs for c in ctx]
+    perm = torch.randperm(pages, generator=g)[: sum(nblk)].tolist()
+    table = torch.zeros(len(lens), max(nblk), dtype=torch.int32)
+    for s, n in enumerate(nblk):
+        table[s, :n] = torch.tensor([perm.pop() for _ in range(n)])
+    pos, slot, tok_seq, start = [], [], [], []
+    for s, (n, c) in enumerate(zip(lens, ctx)):
+        start.append(len(pos))
+        for p in range(c - n, c):
+            pos.append(p)
+            slot.append(int(table[s, p // bs]) * bs + p % bs)
+            tok_seq.append(s)
+
+    class Meta:
+        num_prefill_tokens = sum(n for n in lens if n > 1)
+        num_decode_tokens = sum(1 for n in lens if n == 1)
+        slot_mapping = torch.tensor(slot, device=device)
+        seq_block_tables = table.to(device)
+        seg_start, seg_len, seg_ctx = i32(start, device), i32(list(lens), device), i32(list(ctx), device)
+        max_seg_len = max(lens)
+
+    Meta.tok_seq = i32(tok_seq, device)
+    return Meta, torch.tensor(pos, device=device)
+
+
+@pytest.mark.parametrize("device,dtype", CASES)
+@pytest.mark.parametrize("heads,dim,rot,vdim,rank", [(3, 16, 8, 24, 40), (2, 5, 4, 3, 7), (1, 8, 8, 8, 64), (5, 32, 16, 32, 96)])
+@pytest.mark.parametrize("plant", [None, "far", "page", "own", "past"])
+def test_latent_attention_and_shared_rows(device, dtype, heads, dim, rot, vdim, rank, plant):
+    """A layer that writes rows, then one that only reads them (its own W_uk,
+    W_uv, queries and another scale); prompts in two portions and single
+    tokens.  `plant` makes one cached latent dominate a later query's scores:
+    far back, the last row of a page, the query's own, one past it."""
+    g = torch.Generator().manual_seed(dim)
+    hidden, eps, bs = 40, 1e-5, 8
+    base = 30.0
+    rotc = {"base": base, "dims": rot}
+    mk = lambda own, scale: LatentAttention(
+        hidden, heads, dim, rot, vdim, 0, rank, scale, base, rot, eps, sink=False, out_gate=False,
+        head_gate=True, own_rows=own, device=device, dtype=dtype)
+    a, b = mk(True, 0.3), mk(False, 0.11)
+    assert b.cache_spec() == [] and a.cache_spec() == {"kind": "latent", "row": rank + rot}
+
+    def weights(own):
+        W = {"q": rnd(g, heads * (dim + rot), hidden, s=0.3), "uk": rnd(g, heads * dim, rank, s=0.3),
+             "uv": rnd(g, heads * vdim, rank, s=0.3), "g": rnd(g, heads, hidden, s=0.5), "o": rnd(g, hidden, heads * vdim, s=0.3)}
+        if own:
+            W["dkv"], W["dkv.norm"] = rnd(g, rank + rot, hidden, s=0.3), 1 + 0.2 * rnd(g, rank)
+        return {k: v.to(dtype) for k, v in W.items()}
+
+    Wa, Wb = weights(True), weights(False)
+    a.load(lambda n: Wa[n].to(device), "")
+    b.load(lambda n: Wb[n].to(device), "")
+    T = {0: 50, 1: 21}
+    h = {s: rnd(g, n, hidden).to(dtype) for s, n in T.items()}
+    if plant is not None:
+        # make row j of sequence 0 the one query i picks: h_i strongly along
+        # what scores row j, solved through the first head's weights
+        i, j = 45, {"far": 2, "page": 15, "own": 45, "past": 46}[plant]
+        Wd = {k: v.to(F64) for k, v in Wa.items()}
+        c, _ = O.latent_rows(h[0].to(F64), Wd, "", {"kv_rank": rank, "rot": rotc}, eps)
+        key = Wd["uk"][:dim] @ c[j]
+        d = Wd["q"][:dim].T @ key
+        if plant != "own":
+            h[0][i] = (h[0][i].double() + 30.0 * d / d.norm()).to(dtype)
+    Wad, Wbd = ({k: v.to(F64) for k, v in W.items()} for W in (Wa, Wb))
+    m = {"heads": heads, "dim": dim, "rot_dim": rot, "vdim": vdim, "kv_rank": rank, "rot": rotc}
+    want = {}
+    for s in T:
+        hd = h[s].to(F64)
+        rows = O.latent_rows(hd, Wad, "", m, eps)
+        want[s] = (O.latent_attention(hd, rows, Wad, "", dict(m, scale=0.3)),
+                   O.latent_attention(hd, rows, Wbd, "", dict(m, scale=0.11)))
+    cache = torch.full((20, 1, bs, rank + rot), 3.0, dtype=dtype, device=device)
+    at = {0: 0, 1: 0}
+    steps = [(17, 20), (28, 1), (1, None), (1, None), (3, None)]
+    for n0, n1 in steps:
+        lens = [n0] + ([n1] if n1 else [])
+        for s, n in enumerate(lens):
+            at[s] += n
+        meta, pos = latent_batch(device, bs, lens, [at[s] for s in range(len(lens))] if n1 else [at[0]], 20)
+        # the page assignment of a sequence must not change between steps
+        full, _ = latent_batch(device, bs, [1, 1], [50, 21], 20)
+        meta.seq_block_tables = full.seq_block_tables[: len(lens)].contiguous()
+        meta.slot_mapping = torch.tensor(
+            [int(meta.seq_block_tables[int(s), int(p) // bs]) * bs + int(p) % bs
+             for s, p in zip(meta.tok_seq.tolist(), pos.tolist())], device=device)
+        x = torch.cat([h[s][at[s] - n : at[s]] for s, n in enumerate(lens)]).to(device)
+        for which, layer in enumerate((a, b)):
+            y = layer(x, pos, (cache,), meta).cpu()
+            r = 0
+            for s, n in enumerate(lens):
+                close(y[r : r + n], want[s][which][at[s] - n : at[s]], dtype,
+                      scale=want[s][which].abs().max().item(), tol32=1e-4)
+                r += n
+    assert at == T
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("nsplit", [1, 4])
+def test_latent_rows_kernel_gate(nsplit):
+    """The gate multiplies whole (token, head) rows, with and without context slices."""
+    g = torch.Generator().manual_seed(9)
+    H, row, Dv, bs, dev = 3, 80, 64, 16, "cuda:0"
+    meta, pos = latent_batch(dev, bs, [70, 1, 33], [70, 90, 150], 40)
+    R = 104
+    q = rnd(g, R, H * row, s=0.3).bfloat16().to(dev)
+    cache = rnd(g, 40, 1, bs, row).bfloat16().to(dev)
+    wide = rnd(g, R, H + 5, s=2).bfloat16().to(dev)
+    kw = dict(nsplit=nsplit)
+    args = (q, cache, Dv, meta.seq_block_tables, meta.seg_start, meta.seg_len, meta.seg_ctx, 70, 0.2, H)
+    plain = ops.latent_attention_rows(*args, **kw).float().view(R, H, Dv)
+    gated = ops.latent_attention_rows(*args, gate=wide[:, 5:], **kw).float().view(R, H, Dv)
+    close(gated.cpu(), (plain.cpu().to(F64) * torch.sigmoid(wide[:, 5:].cpu().to(F64))[:, :, None]), torch.bfloat16)
