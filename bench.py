@@ -145,7 +145,27 @@ def main() -> None:
         "roofline; PARTS = engine, kernels or both (benchmarks/bench_streams.py)",
     )
     ap.add_argument("--streams-sizes", default="s,m")
+    ap.add_argument(
+        "--recurrent",
+        nargs="?",
+        const="engine,kernels",
+        default="",
+        metavar="PARTS",
+        help="instead of the serving workload: Garesun (retention, mLSTM and "
+        "shared-latent attention in parallel layers with routed experts) "
+        "beside routed Lopovik and Potatar's recurrent layers at equal size, "
+        "and its kernels beside their counterparts against the roofline; "
+        "PARTS = engine, kernels or both (benchmarks/bench_recurrent.py)",
+    )
+    ap.add_argument("--recurrent-sizes", default="s,m")
     args = ap.parse_args()
+
+    if args.recurrent:
+        sys.path.insert(0, os.path.join(os.path.dirname(os.path.abspath(__file__)), "benchmarks"))
+        import bench_recurrent
+
+        bench_recurrent.main(["--part", args.recurrent, "--sizes", args.recurrent_sizes])
+        return
 
     if args.streams:
         sys.path.insert(0, os.path.join(os.path.dirname(os.path.abspath(__file__)), "benchmarks"))

@@ -29,11 +29,11 @@ def rnd(g, *shape, s=1.0):
     return torch.randn(*shape, generator=g) * s
 
 
-def close(got, want, dtype, scale=None, tol32=2e-5):
+def close(got, want, dtype, scale=None, tol32=2e-5, tol16=2e-2):
     want = want.to(F64)
     ref = max(want.abs().max().item(), 1e-30) if scale is None else scale
     err = (got.detach().double().cpu() - want).abs().max().item() / ref
-    assert err < (tol32 if dtype == torch.float32 else 2e-2), err
+    assert err < (tol32 if dtype == torch.float32 else tol16), err
 
 
 def i32(v, dev):
@@ -167,7 +167,7 @@ def test_squared_relu_experts_both_dispatch_paths(device, dtype, E, top, shared)
     cfg = {"router": {"top": top}, "shared": {"ff": shared} if shared else None}
     want = O.moe_ff(h.to(F64), {k: v.to(F64) for k, v in W.items()}, "", cfg)
     for meta in (_Meta(4), _Meta(0)):  # gathered batches, then every expert on every token
-        close(mlp(h.to(device), meta), want, dtype)
+        close(mlp(h.to(device), meta), want, dtype, tol16=4e-2)
 
 
 # -- matrix-state recurrences ------------------------------------------------------------
@@ -337,7 +337,7 @@ def test_scalar_decay_mixer_whole(device, dtype, kind):
 
     state = torch.full((3, mix.cache_spec()["width"]), 7.0, device=device)
     got = mix(h.to(device), torch.arange(T, device=device), (state,), Meta)
-    close(got, want, dtype, tol32=2e-4)
+    close(got, want, dtype, tol32=2e-4, tol16=4e-2)
 
 
 # -- latent attention with direct queries, a gate per head and shared rows ------------------
@@ -438,7 +438,7 @@ def test_latent_attention_and_shared_rows(device, dtype, heads, dim, rot, vdim, 
             r = 0
             for s, n in enumerate(lens):
                 close(y[r : r + n], want[s][which][at[s] - n : at[s]], dtype,
-                      scale=want[s][which].abs().max().item(), tol32=1e-4)
+                      scale=want[s][which].abs().max().item(), tol32=1e-4, tol16=4e-2)
                 r += n
     assert at == T
 
