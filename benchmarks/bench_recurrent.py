@@ -186,7 +186,7 @@ def part_kernels(sizes) -> None:
             state = torch.zeros(S + 1, ops.matrix_state_width(hr, dr, vr), device=dev)
             add(f"matrix_state_scan, retention ({hr} heads {dr} x {vr}, rotated)", "",
                 timeit(lambda: ops.matrix_state_scan(q, k, v, state, *segs, hr, dr, vr, head_decay=dec, rot=cs,
-                                                     k_scale=0.1), 10), scan_bytes(hr, dr, vr))
+                                                     k_scale=0.1, max_seg_len=seg), 10), scan_bytes(hr, dr, vr))
             add("matrix_state_scan, constant decay + silu, the same sizes", "retention",
                 timeit(lambda: ops.matrix_state_scan(q, k, v, state, *segs, hr, dr, vr, head_decay=dec,
                                                      act_silu=True), 10), scan_bytes(hr, dr, vr))
@@ -201,7 +201,7 @@ def part_kernels(sizes) -> None:
             add(f"matrix_state_scan, mLSTM ({hm} heads {dm} x {vm}, gated)", "",
                 timeit(lambda: ops.matrix_state_scan(qm, km, vmv, state, *segs, hm, dm, vm,
                                                      gates=(zz[:, :hm], zz[:, hm:]), gate_bias=(bi, bfg),
-                                                     gate_cap=15.0, q_scale=0.1), 10), scan_bytes(hm, dm, vm, 1))
+                                                     gate_cap=15.0, q_scale=0.1, max_seg_len=seg), 10), scan_bytes(hm, dm, vm, 1))
             del state
             decm = torch.full((hm,), 0.99, device=dev)
             state = torch.zeros(S + 1, ops.matrix_state_width(hm, dm, vm), device=dev)

@@ -914,12 +914,13 @@ class ScalarDecayMixer(nn.Module):
                 rot = tables[self.rot_key]
             o = ops.matrix_state_scan(
                 q, k, v, state, *seg, *sizes, head_decay=self.head_decay, rot=rot,
-                k_scale=self.dim ** -0.5,
+                k_scale=self.dim ** -0.5, max_seg_len=meta.max_seg_len,
             )
         else:
             o = ops.matrix_state_scan(
                 q, k, v, state, *seg, *sizes, gates=(small[:, : self.heads], small[:, self.heads :]),
                 gate_bias=(self.b_i, self.b_f), gate_cap=self.gate_cap, q_scale=self.dim ** -0.5,
+                max_seg_len=meta.max_seg_len,
             )
         MatrixStateMixer._zero_pad_rows(o, meta)
         return ops.group_rms_norm_gate(

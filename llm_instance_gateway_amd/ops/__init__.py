@@ -1172,7 +1172,7 @@ def matrix_state_scan(
     q, k, v, state, seg_start, seg_len, seg_slot, seg_fresh, heads: int, dim: int,
     vdim: int, decay_pre=None, head_decay=None, bonus=None, act_silu: bool = False,
     gates=None, gate_bias=None, gate_cap: float = 1.0, rot: Optional[torch.Tensor] = None,
-    q_scale: float = 1.0, k_scale: float = 1.0,
+    q_scale: float = 1.0, k_scale: float = 1.0, max_seg_len: int = 0,
 ) -> torch.Tensor:
     """Linear recurrences with one [dim, vdim] fp32 state matrix S per head,
     over the segments of the flat batch; q, k [R, heads*dim] and v
@@ -1191,7 +1191,10 @@ def matrix_state_scan(
         o_t = S^T q_t / (max(|n . q_t|, exp(-m_t)) + 1e-6)
     On the way in, in this order: act_silu applies silu to q, k, v; `rot`
     (fp32 [R, 2n] from rotary_table) turns entries i and i + n of every q and
-    k head; q_scale and k_scale multiply.  state [slots,
+    k head; q_scale and k_scale multiply.  max_seg_len: the step's longest
+    segment; with it, long bf16 portions of the last two forms (without silu)
+    run in chunks of 64 tokens on MFMA tiles where head sizes, rotation and
+    row strides are multiples of 8.  state [slots,
     matrix_state_width] is read unless the segment starts its sequence and
     written back; its layout is private to the implementation.  Returns fp32
     [R, heads*vdim]; rows of no segment are left untouched (undefined)."""
@@ -1231,7 +1234,7 @@ def matrix_state_scan(
             0 if gi is None else gi.stride(0), _ptr(bi), _ptr(bf), float(gate_cap), _ptr(rot), nf,
             float(q_scale), float(k_scale), _ptr(state), state.stride(0),
             _ptr(seg_start), _ptr(seg_len), _ptr(seg_slot), _ptr(seg_fresh), S, heads, dim,
-            vdim, int(bool(act_silu)), _is_f32(q), _stream(),
+            vdim, int(bool(act_silu)), int(max_seg_len), _is_f32(q), _stream(),
         )
         if rc != 0:
             raise RuntimeError("matrix_state_scan: more than 512 key channels per head")

@@ -38,8 +38,13 @@
 // coalesced; in the gated form the running maxima [head][block] follow
 // (ops.matrix_state_width mirrors this).
 // A segment that starts its sequence ignores what the slot held.
+//
+// Long bf16 portions of the constant-decay and gated forms are handed to the
+// chunked MFMA kernel, which reads and writes the same state rows.
 
-#include "elem_types.h"
+#include "matrix_state.h"
+
+#include <climits>
 
 
 // Sum over the 4 or 8 neighbouring lanes that share a value column, through
@@ -58,30 +63,6 @@ LIG_DEVICE float split_sum(float o) {
   if (SPLIT == 8) o += lane_permute<0x141>(o);  // row_half_mirror: lane i <-> 7 - i
   return o;
 }
-
-#define MS_COLS 64  // value columns per workgroup
-
-enum { MS_CONST = 0, MS_BONUS = 1, MS_GATED = 2 };
-
-struct MsArgs {
-  float* out;  // [R, H*Dv]
-  const void *q, *k, *v;
-  long q_stride, k_stride, v_stride;
-  const float* decay_pre;   // [R, H*D]   (bonus form)
-  const float* head_decay;  // [H]        (constant form)
-  const float* bonus;       // [H*D]      (bonus form)
-  const float *gate_i, *gate_f;  // [R, H] views, row stride gate_stride (gated form)
-  long gate_stride;
-  const float *bias_i, *bias_f;  // [H]
-  float gate_cap;
-  const float* cs;  // nullable: [R, 2*nf] cosines | sines of the rotation
-  int nf;
-  float q_scale, k_scale;
-  float* state;
-  long state_stride;
-  const int *seg_start, *seg_len, *seg_slot, *seg_fresh;
-  int H, D, Dv, CB, NB, TT, act_silu;
-};
 
 // Entry i of a query or key head as the recurrence sees it: silu, rotation
 // (entry i paired with i +- nf), constant factor; fp32 throughout.
@@ -123,7 +104,7 @@ __global__ __launch_bounds__(MAXT) void matrix_state_scan_kernel(const MsArgs A)
 
   const int seg = blockIdx.x, h = blockIdx.y, blk = blockIdx.z;
   const int n = A.seg_len[seg];
-  if (n <= 0) return;
+  if (n <= 0 || n < A.len_min || n > A.len_max) return;
   const int r0 = A.seg_start[seg];
   const int tid = threadIdx.x, nt = blockDim.x;
   const int j = tid / MS_SPLIT, s = tid % MS_SPLIT;
@@ -272,20 +253,6 @@ __global__ __launch_bounds__(MAXT) void matrix_state_scan_kernel(const MsArgs A)
   if (GATED && tid == 0) *mrow = m_run;
 }
 
-// Key split and key channels per thread for a head of D key channels: the
-// smallest size class that holds ceil(D / split); kpt 0 when D is too wide.
-static void ms_shape(int D, int* split, int* kpt) {
-  static const int classes[] = {4, 8, 12, 16, 24, 32, 48, 64};
-  *split = D >= 32 ? 8 : 4;
-  const int need = (D + *split - 1) / *split;
-  *kpt = 0;
-  for (int c : classes)
-    if (c >= need) {
-      *kpt = c;
-      break;
-    }
-}
-
 template <typename T, int SPLIT, int KPT, int FORM>
 static void ms_launch(const MsArgs& a, dim3 grid, int threads, size_t smem, hipStream_t stream) {
   if (threads <= 256)
@@ -316,6 +283,11 @@ static void ms_dispatch(const MsArgs& a, int split, int kpt, dim3 grid, int thre
   }
 }
 
+// Portions of at least this many tokens go through the chunked kernel where
+// it serves the shape (bf16, constant-decay or gated form).
+#define MS_CHUNK_MIN 16
+
+// max_seg_len: the longest segment of the step (0: walk every segment).
 // The form follows from the pointers: bonus -> bonus form, gate_i -> gated
 // form, else the constant-decay form.  Returns 0 when launched, 1 when a head
 // is wider than the kernel holds.
@@ -326,7 +298,7 @@ extern "C" int lig_matrix_state_scan(
     const float* bias_i, const float* bias_f, float gate_cap, const float* cs, int nf,
     float q_scale, float k_scale, float* state, long state_stride, const int* seg_start,
     const int* seg_len, const int* seg_slot, const int* seg_fresh, int S, int H,
-    int D, int Dv, int act_silu, int is_f32, hipStream_t stream) {
+    int D, int Dv, int act_silu, int max_seg_len, int is_f32, hipStream_t stream) {
   int split = 4, kpt = 0;
   if (D > 0) ms_shape(D, &split, &kpt);
   if (kpt == 0 || Dv <= 0 || 2 * nf > D) return 1;
@@ -342,11 +314,20 @@ extern "C" int lig_matrix_state_scan(
   const int TT = per_tok * 32 * 4 <= 40 * 1024 ? 32 : (per_tok * 16 * 4 <= 48 * 1024 ? 16 : 8);
   const size_t smem = (size_t)per_tok * TT * sizeof(float);
   const int threads = ((CBw * split + WAVE_SIZE - 1) / WAVE_SIZE) * WAVE_SIZE;
-  const MsArgs a{out, q, k, v, q_stride, k_stride, v_stride, decay_pre, head_decay, bonus,
+  MsArgs a{out, q, k, v, q_stride, k_stride, v_stride, decay_pre, head_decay, bonus,
                  gate_i, gate_f, gate_stride, bias_i, bias_f, gate_cap, cs, nf, q_scale,
                  k_scale, state, state_stride, seg_start, seg_len, seg_slot, seg_fresh,
-                 H, D, Dv, CB, NB, TT, act_silu};
+                 H, D, Dv, CB, NB, TT, act_silu, split, kpt, 1, INT_MAX};
   const dim3 grid(S, H, NB);
+  if (max_seg_len >= MS_CHUNK_MIN && !is_f32 && !act_silu && form != MS_BONUS &&
+      ms_chunks_served(a, form)) {
+    // long portions in chunks, the step's short ones by the walk
+    a.len_min = MS_CHUNK_MIN;
+    ms_chunks_launch(a, form, S, stream);
+    if (S == 1) return 0;
+    a.len_min = 1;
+    a.len_max = MS_CHUNK_MIN - 1;
+  }
 #define LIG_MS_FORM(T)                                                                        \
   if (form == MS_BONUS) ms_dispatch<T, MS_BONUS>(a, split, kpt, grid, threads, smem, stream); \
   else if (form == MS_GATED)                                                                  \

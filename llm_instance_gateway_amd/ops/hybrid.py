@@ -36,7 +36,7 @@ SOURCES = [
     "group_norm.hip", "xielu.hip", "mingru.hip", "attention_general.hip",
     "attention_prefill_tiles.hip", "shift_norm.hip", "latent_attention.hip", "ff_act.hip",
     "attention_latent_rows.hip", "post_norm.hip", "qkv_prep.hip", "attention_mixed_heads.hip",
-    "matrix_state_scan.hip", "attention_mixed_heads_tiles.hip", "hyper_streams.hip",
+    "matrix_state_scan.hip", "matrix_state_chunks.hip", "attention_mixed_heads_tiles.hip", "hyper_streams.hip",
     "routed.hip", "layer_norm.hip", "small_projection.hip",
 ]
 SO_PATH = PKG / "_hybrid.so"
@@ -153,7 +153,7 @@ def _declare(lib: ctypes.CDLL) -> None:
     ms = lib.lig_matrix_state_scan
     ms.argtypes = [
         p, p, l, p, l, p, l, p, p, p, p, p, l, p, p, f, p, i, f, f, p, l, p, p, p, p,
-        i, i, i, i, i, i, p,
+        i, i, i, i, i, i, i, p,
     ]
     ms.restype = ctypes.c_int
     lr = lib.lig_latent_attention_rows

@@ -190,7 +190,8 @@ def scan_in_cuts(device, data, plans, slots, heads, dim, vdim, gated, make_kw):
         a, b = heads * dim, 2 * heads * dim
         o = ops.matrix_state_scan(
             fused[:, :a], fused[:, a:b], fused[:, b : b + heads * vdim], state, i32(start, device),
-            i32(ln, device), i32(sl, device), i32(fresh, device), heads, dim, vdim, **make_kw(rows),
+            i32(ln, device), i32(sl, device), i32(fresh, device), heads, dim, vdim, max_seg_len=max(ln),
+            **make_kw(rows),
         )
         assert o.dtype == torch.float32
         for (s, n), r0 in zip(plan, start):
@@ -211,7 +212,8 @@ CUTS = [[147], [20, 2, 1, 64, 60], [2] * 10 + [127], [1] * 60 + [87], [64, 64, 1
 
 @pytest.mark.parametrize("device,dtype", CASES)
 @pytest.mark.parametrize("heads,dim,vdim,rot", [(3, 10, 6, 4), (2, 32, 64, 32), (1, 40, 65, 16), (2, 8, 130, 0),
-                                                (2, 64, 128, 64), (1, 128, 40, 128), (4, 16, 16, 16)])
+                                                (2, 64, 128, 64), (1, 128, 40, 128), (4, 16, 16, 16),
+                                                (2, 24, 72, 0), (1, 256, 64, 0), (2, 40, 16, 16)])
 def test_retention_scan(device, dtype, heads, dim, vdim, rot):
     """Rotated q and k, scaled k, one decay per head (also exactly 1)."""
     g = torch.Generator().manual_seed(dim)
@@ -261,7 +263,7 @@ def gate_case(kind, g, n, heads):
 
 @pytest.mark.parametrize("device,dtype", CASES)
 @pytest.mark.parametrize("kind", ["plain", "forget", "spike", "keep", "late"])
-@pytest.mark.parametrize("heads,dim,vdim", [(2, 24, 40), (1, 48, 64), (3, 9, 5), (1, 33, 130), (2, 128, 64)])
+@pytest.mark.parametrize("heads,dim,vdim", [(2, 24, 40), (1, 48, 64), (3, 9, 5), (1, 33, 130), (2, 128, 64), (1, 200, 136), (2, 136, 32)])
 def test_mlstm_scan(device, dtype, kind, heads, dim, vdim):
     g = torch.Generator().manual_seed(heads * 100 + dim)
     cap, T, nq = 9.0, {0: 147, 1: 12}, heads * dim
@@ -333,7 +335,7 @@ def test_scalar_decay_mixer_whole(device, dtype, kind):
 
     class Meta:
         seg_start, seg_len, seg_slot, seg_fresh = i32([0], device), i32([T], device), i32([1], device), i32([1], device)
-        num_prefill_tokens, num_decode_tokens = T, 0
+        num_prefill_tokens, num_decode_tokens, max_seg_len = T, 0, T
 
     state = torch.full((3, mix.cache_spec()["width"]), 7.0, device=device)
     got = mix(h.to(device), torch.arange(T, device=device), (state,), Meta)
