@@ -23,7 +23,8 @@ class LayerSpec:
     (the normalised key/value latent followed by the shared rotated key
     part), or nothing when it reads another layer's rows ('kv_from').  'wkv' keeps a matrix state per head and the previous token's
     input row; 'retention' and 'mlstm' keep a matrix state per head (the
-    latter with a normaliser vector and a running maximum); 'parallel' keeps paged K/V for its attention branch and a
+    latter with a normaliser vector and a running maximum), 'delta' one beside
+    the last inputs of its short convolutions; 'parallel' keeps paged K/V for its attention branch and a
     matrix state per head for its recurrent branch.  `shift` says the mixer's input is blended with the previous
     token's, which costs one fp32 row of model width per sequence."""
 
@@ -80,8 +81,9 @@ class ModelConfig:
     # one stream without them is the ordinary residual.
     residual_streams: int = 1
     hyper_connections: bool = False
-    # Factor on the embedding rows.
+    # Factor on the embedding rows, and on the logits.
     embed_scale: float = 1.0
+    logit_scale: float = 1.0
     # Entries per layer of a second token table whose row enters the residual
     # after every layer (0 = no such table).
     token_side_dim: int = 0
@@ -141,6 +143,11 @@ class ModelConfig:
             elif s.type == "mlstm":
                 # matrix, normaliser vector and running maximum per head
                 total += s.mixer["heads"] * (s.mixer["dim"] * (s.mixer["vdim"] + 1) + 1)
+            elif s.type == "delta":
+                # matrix per head, and the convolutions' last inputs
+                m = s.mixer
+                total += m["heads"] * m["dim"] * m["vdim"]
+                total += (m["conv"] - 1) * (2 * m["kv_heads"] * m["dim"] + m["heads"] * m["vdim"])
             elif s.type == "parallel":
                 right = s.mixer["right"]
                 total += right["heads"] * right["dim"] * right["vdim"]

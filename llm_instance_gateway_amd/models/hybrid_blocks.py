@@ -16,13 +16,15 @@ arguments, so another model family can assemble them differently.
     key/value attention and its feed-forwards.
   * `NormedRotaryAttention` — q/k norms before or after a partial rotation in
     either pair layout, chunked or sliding-window visibility, softmax (with
-    an optional sink) or unnormalised sigmoid weights, distance bias, head
-    mixing, per-head output gate.
+    an optional sink) or unnormalised sigmoid weights, soft-capped scores,
+    distance bias, head mixing, per-head output gate.
   * `MatrixStateMixer`, `GeluMLP` — matrix-state recurrences.
-  * `GatedReluMLP`, `GroupRoutedExpertsMLP` — gated feed-forward and routed
+  * `GatedMLP`, `GroupRoutedExpertsMLP` — gated feed-forward and routed
     experts with a softmax router, group-limited choice and identity experts.
   * `ScalarDecayMixer` — matrix-state recurrences whose decay is one number
     per head: fixed (retention) or gated per token (mLSTM).
+  * `GatedDeltaMixer` — the gated delta rule behind short convolutions: every
+    write corrects what the matrix state holds under the token's key.
   * `ReluSquaredExpertsMLP` — routed squared-ReLU experts beside a shared one.
   * `TokenTableGate` — a per-layer token table that enters the residual
     through a gate and a norm.
@@ -249,6 +251,8 @@ class LatentAttention(nn.Module):
     kernel, which commutes with W_uv).  Rotation is interleaved pairs over
     the first `rot_dims` entries of the rotated part.
 
+    window > 0: a query sees itself and the window - 1 tokens before it.
+    rot_scaling: band-wise frequency scaling (`ops.rotary_inv_freq`).
     q_rank 0: queries are projected directly, without a normed query latent.
     own_rows False: the layer caches nothing and has no down-projection; the
     cache handed to it holds another layer's rows.
@@ -261,7 +265,8 @@ class LatentAttention(nn.Module):
         self, hidden: int, heads: int, dim: int, rot_dim: int, vdim: int, q_rank: int,
         kv_rank: int, scale: float, rot_base: float, rot_dims: int, eps: float,
         sink: bool = True, out_gate: bool = True, head_gate: bool = False,
-        own_rows: bool = True, device="cpu", dtype=torch.bfloat16,
+        own_rows: bool = True, window: int = 0, rot_scaling: Optional[dict] = None,
+        device="cpu", dtype=torch.bfloat16,
     ) -> None:
         super().__init__()
         assert 0 <= rot_dims <= rot_dim and rot_dims % 2 == 0
@@ -270,6 +275,7 @@ class LatentAttention(nn.Module):
         self.q_rank, self.kv_rank = q_rank, kv_rank
         self.scale, self.eps = float(scale), float(eps)
         self.out_gate, self.head_gate, self.own_rows = out_gate, head_gate, own_rows
+        self.window = int(window)
         self.row = kv_rank + rot_dim  # one cache row
         self.n_out = heads * vdim
         s = 1.0 / math.sqrt(hidden)
@@ -298,7 +304,8 @@ class LatentAttention(nn.Module):
         )
         self.w_o = _param((hidden, heads * vdim), device, dtype, 1.0 / math.sqrt(heads * vdim))
         self.register_buffer(
-            "inv_freq", ops.rotary_inv_freq(rot_base, rot_dims, device), persistent=False
+            "inv_freq", ops.rotary_inv_freq(rot_base, rot_dims, device, scaling=rot_scaling),
+            persistent=False,
         )
 
     def cache_spec(self):
@@ -372,12 +379,13 @@ class LatentAttention(nn.Module):
             ops.latent_attention_rows(
                 qa, lat_cache, Rk, meta.seq_block_tables, meta.seg_start, meta.seg_len,
                 meta.seg_ctx, meta.max_seg_len, self.scale, H, sink=self.sink, out=o,
-                gate=head_gate,
+                gate=head_gate, window=self.window,
             )
         else:
             o = ops.paged_attention_general(
                 qa, lat_cache, v_view, meta.seq_block_tables, meta.tok_seq, positions,
                 self.scale, H, sink=self.sink, gate=head_gate, gate_per_head=self.head_gate,
+                window=self.window,
             )
         # values: per head o_lat @ W_uv, heads concatenated in place
         if out is None:
@@ -488,8 +496,10 @@ class NormedRotaryAttention(nn.Module):
         weights; "none".
       * rot_dims entries of every head are rotated; rot_layout "half" pairs
         entry i with i + rot_dims/2, "interleaved" pairs 2i with 2i + 1;
-        rot_scale divides every frequency (linear position scaling);
-        0 = no rotation.
+        rot_scale divides every frequency (linear position scaling),
+        rot_scaling scales them band by band (`ops.rotary_inv_freq`); 0 = no
+        rotation.
+      * softcap > 0: scores are bent by softcap * tanh(score / softcap).
       * window: a query sees itself and the window - 1 tokens before it
         (0 = no window; may be combined with chunk).
       * weights "softmax", optionally with a zero-score sink in the
@@ -521,13 +531,17 @@ class NormedRotaryAttention(nn.Module):
         dist_rows: int = 0, dist_far: float = 0.0, talk: bool = False,
         rot_layout: str = "half", rot_scale: float = 1.0, window: int = 0,
         weights: str = "softmax", score_bias: bool = False, sink: bool = False,
-        head_gate: bool = False, device="cpu", dtype=torch.bfloat16,
+        head_gate: bool = False, softcap: float = 0.0, rot_scaling: Optional[dict] = None,
+        device="cpu", dtype=torch.bfloat16,
     ) -> None:
         super().__init__()
         assert heads % kv_heads == 0 and qk_norm in ("none", "row", "head", "head_post")
         assert rot_layout in ("half", "interleaved") and weights in ("softmax", "sigmoid")
         assert not (score_bias and weights != "sigmoid") and not (sink and weights != "softmax")
-        assert not ((dist_rows > 0 or talk) and (window > 0 or weights == "sigmoid" or sink or head_gate))
+        assert not (
+            (dist_rows > 0 or talk)
+            and (window > 0 or weights == "sigmoid" or sink or head_gate or softcap > 0)
+        )
         assert values in ("proj", "key") and (values == "proj" or vdim == dim)
         assert 0 <= rot_dims <= dim and rot_dims % 2 == 0
         self.heads, self.kv_heads, self.dim, self.vdim = heads, kv_heads, dim, vdim
@@ -537,6 +551,7 @@ class NormedRotaryAttention(nn.Module):
         self.nv = kv_heads * vdim if values == "proj" else 0
         self.n_in = self.nq + self.nk + self.nv
         self.window, self.weights, self.rot_layout = int(window), weights, rot_layout
+        self.softcap = float(softcap)
         # gate rows follow q | k | v; the fused weight is padded with zero rows
         # to a multiple of 8 so that rows of the projection stay 16-byte aligned
         self.n_gate = heads if head_gate else 0
@@ -582,7 +597,8 @@ class NormedRotaryAttention(nn.Module):
         self.refresh_tables()
         self.register_buffer(
             "inv_freq",
-            ops.rotary_inv_freq(rot_base, rot_dims, device, rot_scale) if rot_dims > 0 else None,
+            ops.rotary_inv_freq(rot_base, rot_dims, device, rot_scale, rot_scaling)
+            if rot_dims > 0 else None,
             persistent=False,
         )
 
@@ -679,6 +695,7 @@ class NormedRotaryAttention(nn.Module):
         kw = dict(
             chunk=self.chunk, window=self.window, weights=self.weights,
             score_bias=self.score_bias, sink=self.sink, gate_per_head=gate is not None,
+            softcap=self.softcap,
         )
         if (
             np_ > 0
@@ -929,6 +946,82 @@ class ScalarDecayMixer(nn.Module):
         )
 
 
+class GatedDeltaMixer(nn.Module):
+    """The gated delta rule (`ops.gated_delta_scan`): one [dim, vdim] fp32
+    state matrix per value head that decays by one number per token and whose
+    write is the difference between the value and what the state holds under
+    the token's key.  q and k have kv_heads heads, shared by groups of value
+    heads; q, k and v pass a short causal convolution per channel and silu
+    (`ops.short_conv_silu`, whose last inputs are a second state row), q and k
+    become unit vectors per head, q is scaled by dim^-1/2.  Every head's output
+    is divided by its root mean square, times a weight shared by the heads,
+    times silu(gate).
+
+    Rows of w_in: q | k | v | gate.  `w_small` holds the rows of the write
+    strength and of the decay, [b | a]; their logits are computed in fp32.
+    """
+
+    UNIT_EPS = 1e-6  # inside the root of the unit norms
+
+    def __init__(
+        self, hidden: int, heads: int, kv_heads: int, dim: int, vdim: int, taps: int, eps: float,
+        device="cpu", dtype=torch.bfloat16,
+    ) -> None:
+        super().__init__()
+        assert heads % kv_heads == 0 and taps >= 1
+        self.heads, self.kv_heads, self.dim, self.vdim = heads, kv_heads, dim, vdim
+        self.taps, self.eps = taps, float(eps)
+        self.nk, self.nv = kv_heads * dim, heads * vdim
+        self.channels = 2 * self.nk + self.nv
+        s = 1.0 / math.sqrt(hidden)
+        self.w_in = _param((self.channels + self.nv, hidden), device, dtype, s)
+        self.w_conv = _param((taps, self.channels), device, dtype, 1.0 / math.sqrt(taps))
+        self.w_small = _param((2 * heads, hidden), device, dtype, s)
+        # they enter the recurrence: fp32
+        f32 = dict(device=device, dtype=torch.float32)
+        self.log_rate = nn.Parameter(torch.zeros(heads, **f32), requires_grad=False)
+        self.dt_bias = nn.Parameter(torch.full((heads,), -4.0, **f32), requires_grad=False)
+        # the weight of one head, repeated for every head
+        self.norm = _param((self.nv,), device, dtype, None)
+        with torch.no_grad():
+            self.norm.fill_(1.0)
+        self.w_o = _param((hidden, self.nv), device, dtype, 1.0 / math.sqrt(self.nv))
+
+    def cache_spec(self):
+        return [
+            {"kind": "state", "width": (self.taps - 1) * self.channels},
+            {"kind": "state", "width": ops.matrix_state_width(self.heads, self.dim, self.vdim)},
+        ]
+
+    def load(self, get, prefix: str) -> None:
+        with torch.no_grad():
+            self.w_in.copy_(torch.cat([get(prefix + n) for n in "qkvg"], dim=0))
+            self.w_conv.copy_(torch.cat([get(prefix + n + ".conv") for n in "qkv"], dim=0).t())
+            self.w_small.copy_(torch.cat([get(prefix + "b"), get(prefix + "a")], dim=0))
+            self.log_rate.copy_(get(prefix + "A_log").float())
+            self.dt_bias.copy_(get(prefix + "dt_bias").float())
+            self.norm.copy_(get(prefix + "norm").repeat(self.heads))
+            self.w_o.copy_(get(prefix + "o"))
+
+    def forward(self, h, positions, cache, meta):
+        conv_state, mat_state = cache
+        a, b, H = self.nk, 2 * self.nk, self.heads
+        seg = (meta.seg_start, meta.seg_len, meta.seg_slot, meta.seg_fresh)
+        small = ops.small_projection(h, self.w_small)
+        proj = _mm(h, self.w_in)
+        qkv = ops.short_conv_silu(
+            proj[:, : self.channels], self.w_conv, conv_state, *seg, meta.max_seg_len
+        )
+        o = ops.gated_delta_scan(
+            qkv[:, :a], qkv[:, a:b], qkv[:, b:], (small[:, :H], small[:, H:]), self.log_rate,
+            self.dt_bias, mat_state, *seg, H, self.kv_heads, self.dim, self.vdim,
+            q_scale=self.dim ** -0.5, unit_eps=self.UNIT_EPS, max_seg_len=meta.max_seg_len,
+        )
+        MatrixStateMixer._zero_pad_rows(o, meta)
+        g = ops.group_rms_norm_gate(o, proj[:, self.channels :], self.norm, self.vdim, "silu", self.eps)
+        return _mm(g, self.w_o)
+
+
 class GeluMLP(nn.Module):
     """down(gelu(up h)) with the exact (erf) gelu."""
 
@@ -946,11 +1039,14 @@ class GeluMLP(nn.Module):
         return _mm(ops.gelu_erf(_mm(h, self.w_up)), self.w_down)
 
 
-class GatedReluMLP(nn.Module):
-    """down(relu(gate h) * (up h)); gate and up are one fused GEMM."""
+class GatedMLP(nn.Module):
+    """down(act(gate h) * (up h)), act "relu" or "gelu_tanh"; gate and up are
+    one fused GEMM."""
 
-    def __init__(self, hidden: int, ff: int, device="cpu", dtype=torch.bfloat16) -> None:
+    def __init__(self, hidden: int, ff: int, act: str = "relu", device="cpu", dtype=torch.bfloat16) -> None:
         super().__init__()
+        assert act in ("relu", "gelu_tanh")
+        self.act = act
         self.w13 = _param((2 * ff, hidden), device, dtype, 1.0 / math.sqrt(hidden))
         self.w_down = _param((hidden, ff), device, dtype, 1.0 / math.sqrt(ff))
 
@@ -960,7 +1056,7 @@ class GatedReluMLP(nn.Module):
             self.w_down.copy_(get(prefix + "down"))
 
     def forward(self, h, meta=None):
-        return _mm(ops.glu_act(_mm(h, self.w13), "relu"), self.w_down)
+        return _mm(ops.glu_act(_mm(h, self.w13), self.act), self.w_down)
 
 
 def expert_dispatch_plan(idx: torch.Tensor, experts: int):

@@ -92,7 +92,20 @@ def _garesun_config(raw: dict, path: str) -> ModelConfig:
     return config_from_json(raw, path)
 
 
+def _daberax_factory(cfg, device, dtype, tp):
+    from .daberax import DaberaxForCausalLM
+
+    return DaberaxForCausalLM(cfg, device=device, dtype=dtype, tp=tp)
+
+
+def _daberax_config(raw: dict, path: str) -> ModelConfig:
+    from .daberax import config_from_json
+
+    return config_from_json(raw, path)
+
+
 register_architecture("llama", None, _llama_factory)
+register_architecture("daberax", _daberax_config, _daberax_factory)
 register_architecture("garesun", _garesun_config, _garesun_factory)
 register_architecture("vemenex", _vemenex_config, _vemenex_factory)
 register_architecture("potatar", _potatar_config, _potatar_factory)

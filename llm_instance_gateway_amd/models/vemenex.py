@@ -40,7 +40,7 @@ import torch.nn as nn
 
 from .. import ops
 from .config import LayerSpec, ModelConfig
-from .hybrid_blocks import GatedReluMLP, GroupRoutedExpertsMLP, NormedRotaryAttention, _param
+from .hybrid_blocks import GatedMLP, GroupRoutedExpertsMLP, NormedRotaryAttention, _param
 
 MIXERS = ("attention", "attention_2")
 
@@ -115,7 +115,7 @@ def _attention(kind: str, hidden: int, m: dict, eps: float, device, dtype) -> No
 
 def _feed_forward(hidden: int, mlp: dict, device, dtype):
     if mlp.get("kind", "dense") == "dense":
-        return GatedReluMLP(hidden, int(mlp["ff"]), device=device, dtype=dtype)
+        return GatedMLP(hidden, int(mlp["ff"]), "relu", device=device, dtype=dtype)
     r = mlp["router"]
     grp = r.get("groups") or {}
     return GroupRoutedExpertsMLP(

@@ -377,20 +377,27 @@ def group_norm(residual, w, eps: float, groups: int) -> torch.Tensor:
     return torch_ref.group_norm(residual, w, eps, groups, w.dtype)
 
 
-def post_add_pre_norm(residual, y, w_post, w_pre, eps: float, groups: int):
+def post_add_pre_norm(residual, y, w_post, w_pre, eps: float, groups: int, rounded: bool = False):
     """residual += group_norm(y) * w_post (in place); returns
-    group_norm(residual) * w_pre in y's dtype (None when w_pre is None)."""
+    group_norm(residual) * w_pre in y's dtype (None when w_pre is None).
+    rounded (without w_pre): returns the new residual in y's dtype, which is
+    what the next sub-layer reads in stacks without input norms."""
     R, H = residual.shape
     assert residual.dtype == torch.float32 and y.shape == residual.shape
+    assert not (rounded and w_pre is not None)
+    if rounded and y.dtype == torch.float32:
+        post_add_pre_norm(residual, y, w_post, None, eps, groups)
+        return residual
     if _use_hybrid(residual):
         assert y.is_contiguous() and residual.is_contiguous()
-        out = None if w_pre is None else torch.empty_like(y)
+        out = None if w_pre is None and not rounded else torch.empty_like(y)
         _hl().lig_post_add_pre_norm(
             _ptr(out), _ptr(residual), _ptr(y), _ptr(w_post), _ptr(w_pre),
             float(eps), R, H, groups, _is_f32(y), _stream(),
         )
         return out
-    return torch_ref.post_add_pre_norm(residual, y, w_post, w_pre, eps, groups)
+    out = torch_ref.post_add_pre_norm(residual, y, w_post, w_pre, eps, groups)
+    return residual.to(y.dtype) if rounded else out
 
 
 def xielu(x: torch.Tensor, a_pos: float, a_neg: float) -> torch.Tensor:
@@ -482,7 +489,7 @@ def paged_attention_general(
     num_heads: int, gate=None, temp_coef: float = 0.0, temp_every: float = 1.0,
     out: Optional[torch.Tensor] = None, sink: Optional[torch.Tensor] = None,
     chunk: int = 0, window: int = 0, score_bias: Optional[torch.Tensor] = None,
-    weights: str = "softmax", gate_per_head: bool = False,
+    weights: str = "softmax", gate_per_head: bool = False, softcap: float = 0.0,
 ) -> torch.Tensor:
     """Causal paged attention for any key/value head sizes; token r of the
     flat batch attends keys 0..positions[r] of sequence tok_seq[r].  Optional
@@ -494,7 +501,8 @@ def paged_attention_general(
     window > 0: only keys j with p - j < window.  weights "sigmoid": every
     visible key weighs sigmoid(score + score_bias[head]) (fp32 [heads],
     optional) and nothing is normalised.  gate_per_head: gate is [R, heads],
-    one logistic gate per head."""
+    one logistic gate per head.  softcap > 0: score <- softcap *
+    tanh(score / softcap), after the scale and ahead of the weights."""
     assert weights in ("softmax", "sigmoid") and (weights == "sigmoid" or score_bias is None)
     if _use_hybrid(q):
         nb, G, bs, D = k_cache.shape
@@ -525,13 +533,13 @@ def paged_attention_general(
             _ptr(sink), float(scale), float(temp_coef), ev, ev_int, R, num_heads,
             G, D, Dv, v_row, bs, int(chunk), int(window), _ptr(score_bias),
             int(weights == "sigmoid"), int(bool(gate_per_head and gate is not None)),
-            _is_f32(q), _stream(),
+            float(softcap), _is_f32(q), _stream(),
         )
         return out
     res = torch_ref.paged_attention_general(
         q, k_cache, v_cache, block_tables, tok_seq, positions, scale, num_heads,
         gate, temp_coef, temp_every, sink, chunk, window, score_bias, weights,
-        gate_per_head,
+        gate_per_head, softcap,
     )
     if out is not None:
         out.copy_(res)
@@ -595,7 +603,7 @@ def paged_attention_prefill_tiles(
     temp_every: float = 1.0, out: Optional[torch.Tensor] = None,
     sink: Optional[torch.Tensor] = None, chunk: int = 0, window: int = 0,
     score_bias: Optional[torch.Tensor] = None, weights: str = "softmax",
-    gate_per_head: bool = False,
+    gate_per_head: bool = False, softcap: float = 0.0,
 ) -> torch.Tensor:
     """Prompt-partition attention on MFMA tiles for any head sizes the kernel
     takes (`tiled_prefill_supported`): q [Tp, H*D] (strided view allowed) are
@@ -604,8 +612,8 @@ def paged_attention_prefill_tiles(
     tile_qstart name the 64-row query tiles.  Temperature, sigmoid gate and
     softmax sink are fused; v_cache may view the head of k_cache's rows; chunk
     > 0 restricts every row to the keys of its own chunk, window > 0 to the
-    last `window` keys up to its own.  weights "sigmoid", score_bias and
-    gate_per_head as in `paged_attention_general`.  GPU only."""
+    last `window` keys up to its own.  weights "sigmoid", score_bias,
+    gate_per_head and softcap as in `paged_attention_general`.  GPU only."""
     assert weights in ("softmax", "sigmoid") and (weights == "sigmoid" or score_bias is None)
     nb, G, bs, D = k_cache.shape
     Dv = v_cache.shape[-1]
@@ -635,7 +643,7 @@ def paged_attention_prefill_tiles(
         _ptr(block_tables), float(scale), float(temp_coef), ev, ev_int,
         tile_seq.shape[0], num_heads, G, D, Dv, v_row, bs, block_tables.shape[1],
         int(chunk), int(window), _ptr(score_bias), int(weights == "sigmoid"),
-        int(bool(gate_per_head and gate is not None)), _stream(),
+        int(bool(gate_per_head and gate is not None)), float(softcap), _stream(),
     )
     if rc != 0:
         raise RuntimeError("paged_attention_prefill_tiles: shape or alignment not served")
@@ -674,7 +682,7 @@ def latent_attention_rows(
     q, cache, v_dim: int, block_tables, seg_start, seg_len, seg_ctx, max_seg_len: int,
     scale: float, num_heads: int, sink: Optional[torch.Tensor] = None,
     out: Optional[torch.Tensor] = None, nsplit: int = 0,
-    gate: Optional[torch.Tensor] = None,
+    gate: Optional[torch.Tensor] = None, window: int = 0,
 ) -> torch.Tensor:
     """Causal multi-query attention of every segment of the step (prompt
     portions and single tokens alike) over the paged latent cache
@@ -685,7 +693,8 @@ def latent_attention_rows(
     this step.  Rows of no segment are left untouched.  nsplit > 1 cuts every
     tile's visible keys into that many slices run by separate workgroups and
     merged afterwards (0: chosen from the row count and the longest context
-    the block tables can hold).  GPU, bf16."""
+    the block tables can hold).  window > 0: a token at position p sees keys
+    j with p - j < window.  GPU, bf16."""
     nb, G, bs, row = cache.shape
     R = q.shape[0]
     assert G == 1 and q.is_cuda and q.dtype == torch.bfloat16 and cache.dtype == q.dtype
@@ -702,7 +711,10 @@ def latent_attention_rows(
         out = torch.empty(R, num_heads * v_dim, dtype=q.dtype, device=q.device)
     assert out.shape == (R, num_heads * v_dim) and out.is_contiguous() and out.dtype == q.dtype
     if nsplit <= 0:
-        nsplit = latent_rows_nsplit(R, S, num_heads, block_tables.shape[1] * bs)
+        visible = block_tables.shape[1] * bs
+        if window > 0:  # a 64-row tile sees the window and its own tokens
+            visible = min(visible, window + 64)
+        nsplit = latent_rows_nsplit(R, S, num_heads, visible)
     scratch = None
     if nsplit > 1:
         scratch = split_scratch(q.device, R * num_heads * nsplit * (v_dim + 4))
@@ -710,7 +722,7 @@ def latent_attention_rows(
         _ptr(out), _ptr(q), _ptr(cache), _ptr(sink), _ptr(gate),
         0 if gate is None else gate.stride(0), _ptr(seg_start), _ptr(seg_len),
         _ptr(seg_ctx), _ptr(block_tables), block_tables.shape[1], float(scale), S,
-        int(max_seg_len), num_heads, row, v_dim, bs, int(nsplit), _ptr(scratch), _stream(),
+        int(max_seg_len), num_heads, row, v_dim, bs, int(window), int(nsplit), _ptr(scratch), _stream(),
     )
     if rc != 0:
         raise RuntimeError("latent_attention_rows: shape or alignment not served")
@@ -1245,6 +1257,95 @@ def matrix_state_scan(
     )
 
 
+def short_conv_silu(
+    x: torch.Tensor, w: torch.Tensor, state: torch.Tensor, seg_start, seg_len, seg_slot, seg_fresh,
+    max_seg_len: int,
+) -> torch.Tensor:
+    """Causal convolution over time with one filter per channel, then silu:
+    out[t] = silu(sum_j w[j] * x[t - (taps - 1) + j]); x [R, C] (may be a
+    column block), w [taps, C] in x's dtype, row j weighing the input taps -
+    1 - j tokens back.  state [slots, (taps - 1) * C] fp32 holds every
+    sequence's last taps - 1 inputs, oldest first; it stands ahead of a
+    segment's first row (zeros when the segment starts its sequence) and then
+    takes the segment's last inputs.  max_seg_len: the longest segment.
+    Returns contiguous [R, C]; rows of no segment are left untouched
+    (undefined)."""
+    R, C = x.shape
+    taps = w.shape[0]
+    assert w.shape == (taps, C) and w.dtype == x.dtype and state.dtype == torch.float32
+    assert state.shape[1] == (taps - 1) * C
+    if _use_hybrid(x):
+        assert x.stride(1) == 1 and w.is_contiguous() and state.is_contiguous()
+        out = torch.empty(R, C, dtype=x.dtype, device=x.device)
+        rc = _hl().lig_short_conv_silu(
+            _ptr(out), _ptr(x), x.stride(0), _ptr(w), _ptr(state), state.shape[1],
+            _ptr(seg_start), _ptr(seg_len), _ptr(seg_slot), _ptr(seg_fresh), seg_start.shape[0],
+            int(max_seg_len), C, taps, _is_f32(x), _stream(),
+        )
+        if rc != 0:
+            raise RuntimeError("short_conv_silu: shape not served")
+        return out
+    return torch_ref.short_conv_silu(x, w, state, seg_start, seg_len, seg_slot, seg_fresh)
+
+
+def gated_delta_scan(
+    q, k, v, gates, log_rate, bias, state, seg_start, seg_len, seg_slot, seg_fresh,
+    heads: int, kv_heads: int, dim: int, vdim: int, q_scale: float = 1.0,
+    unit_eps: float = 1e-6, max_seg_len: int = 0,
+) -> torch.Tensor:
+    """The gated delta rule with one [dim, vdim] fp32 state matrix S per head,
+    over the segments of the flat batch (in row order).  q, k [R,
+    kv_heads*dim] and v [R, heads*vdim] may be column-block views; head h
+    reads q/k head h // (heads // kv_heads).  gates = (b, a), fp32 [R, heads]
+    each with one row stride; log_rate, bias fp32 [heads]:
+
+        q <- q_scale * q / sqrt(sum q^2 + unit_eps);  k likewise, unscaled
+        g = exp(-exp(log_rate) softplus(a + bias)),  beta = sigmoid(b)
+        S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+
+    max_seg_len: the step's longest segment; with it, long bf16 portions run
+    in chunks of 64 tokens on MFMA tiles where head sizes and row strides are
+    multiples of 8 and dim is at most 256.  state [slots,
+    matrix_state_width(heads, dim, vdim)] is read unless the segment starts
+    its sequence and written back; its layout is private to the
+    implementation.  Returns fp32 [R, heads*vdim]; rows of no segment are left
+    untouched (undefined)."""
+    b, a = gates
+    R = q.shape[0]
+    assert state.dtype == torch.float32 and heads % kv_heads == 0
+    if _use_hybrid(q):
+        assert q.shape[1] == kv_heads * dim and k.shape[1] == kv_heads * dim and v.shape[1] == heads * vdim
+        assert q.stride(1) == 1 and k.stride(1) == 1 and v.stride(1) == 1
+        assert q.dtype == k.dtype == v.dtype
+        assert state.is_contiguous() and state.shape[1] == matrix_state_width(heads, dim, vdim)
+        for g in gates:
+            assert g.dtype == torch.float32 and g.shape == (R, heads) and g.stride(1) == 1
+            assert g.stride(0) == b.stride(0)
+        for t in (log_rate, bias):
+            assert t.dtype == torch.float32 and t.shape == (heads,) and t.is_contiguous()
+        S = seg_start.shape[0]
+        out = torch.empty(R, heads * vdim, dtype=torch.float32, device=q.device)
+        scratch = None
+        if max_seg_len > 1 and q.dtype == torch.bfloat16:
+            scratch = torch.empty(
+                _hl().lig_gated_delta_scratch(R, S, heads), dtype=torch.uint8, device=q.device
+            )
+        rc = _hl().lig_gated_delta_scan(
+            _ptr(out), _ptr(q), q.stride(0), _ptr(k), k.stride(0), _ptr(v), v.stride(0), _ptr(b),
+            _ptr(a), b.stride(0), _ptr(log_rate), _ptr(bias), float(q_scale), float(unit_eps),
+            _ptr(state), state.stride(0), _ptr(seg_start), _ptr(seg_len), _ptr(seg_slot),
+            _ptr(seg_fresh), S, heads, kv_heads, dim, vdim, int(max_seg_len), _ptr(scratch),
+            _is_f32(q), _stream(),
+        )
+        if rc != 0:
+            raise RuntimeError("gated_delta_scan: more than 512 key channels per head")
+        return out
+    return torch_ref.gated_delta_scan(
+        q, k, v, b, a, log_rate, bias, state, seg_start, seg_len, seg_slot, seg_fresh, heads,
+        kv_heads, dim, vdim, q_scale, unit_eps,
+    )
+
+
 def group_rms_norm_gate(
     o, gate, w, group: int, gate_act: str, eps: float, out: Optional[torch.Tensor] = None
 ) -> torch.Tensor:
@@ -1487,13 +1588,14 @@ def add_layer_norm(x, w, eps: float, y=None, w_y=None):
     return torch_ref.add_layer_norm(x, w, eps, y, w_y)
 
 
-_GLU_KINDS = {"relu": 0, "clamped": 1}
+_GLU_KINDS = {"relu": 0, "clamped": 1, "gelu_tanh": 2}
 
 
 def glu_act(x: torch.Tensor, kind: str, limit: float = 0.0, alpha: float = 1.0) -> torch.Tensor:
     """[rows, 2F] fused (gate | up) -> [rows, F].  "relu": relu(gate) * up.
     "clamped": g = min(gate, limit), u = clamp(up, -limit, limit),
-    g * sigmoid(alpha * g) * (u + 1)."""
+    g * sigmoid(alpha * g) * (u + 1).  "gelu_tanh": gelu(gate) * up, the tanh
+    form of gelu."""
     k = _GLU_KINDS[kind]
     if _use_hybrid(x):
         assert x.is_contiguous() and x.dim() == 2 and x.shape[1] % 2 == 0

@@ -26,6 +26,9 @@
 // window > 0 restricts a query at position p to keys j with p - j < window
 // (itself and the window - 1 tokens before it).
 //
+// softcap > 0 bends every score, s <- softcap * tanh(s / softcap), ahead of
+// the weights.
+//
 // sigmoid_weights: instead of a softmax every visible key weighs
 // sigmoid(score + score_bias[h]) (score_bias nullable, fp32 per head); the
 // weights are not normalised over the keys.  gate_per_head: the output gate
@@ -61,7 +64,8 @@ __global__ __launch_bounds__(WAVE_SIZE * NW) void paged_attention_general_kernel
     const T* __restrict__ gate, long gate_stride, const float* __restrict__ sink,
     float scale, float temp_coef, float temp_every, int temp_every_int, int H,
     int G, int D, int Dv, int v_row, int BS, int chunk, int window,
-    const float* __restrict__ score_bias, int sigmoid_weights, int gate_per_head) {
+    const float* __restrict__ score_bias, int sigmoid_weights, int gate_per_head,
+    float softcap) {
   extern __shared__ __align__(16) float smem[];
   const int Dpad = (D + 1) & ~1;
   float* q_s = smem;                                   // [HB][Dpad]
@@ -160,7 +164,9 @@ __global__ __launch_bounds__(WAVE_SIZE * NW) void paged_attention_general_kernel
       p[hh] = 0.f;
       alpha[hh] = 1.f;
       if (active) {
-        const float score = valid ? dot[hh] * sc : -INFINITY;
+        float score = dot[hh] * sc;
+        if (softcap > 0.f) score = softcap * tanhf(score / softcap);
+        if (!valid) score = -INFINITY;
         if (sigmoid_weights) {
           p[hh] = valid ? sigmoid_f32(score + sb[hh]) : 0.f;
         } else {
@@ -417,7 +423,7 @@ void lig_paged_attention_general(
     long gate_stride, const float* sink, float scale, float temp_coef,
     float temp_every, int temp_every_int, int R, int H, int G, int D, int Dv,
     int v_row, int BS, int chunk, int window, const float* score_bias,
-    int sigmoid_weights, int gate_per_head, int is_f32, hipStream_t s) {
+    int sigmoid_weights, int gate_per_head, float softcap, int is_f32, hipStream_t s) {
   if (R <= 0) return;
   // heads of one key/value head that a wave serves together: as many as
   // divide the group, but fewer while that would leave the chip short of
@@ -439,7 +445,7 @@ void lig_paged_attention_general(
                      max_blocks, tok_seq, positions, (const T*)gate,            \
                      gate_stride, sink, scale, temp_coef, temp_every,           \
                      temp_every_int, H, G, D, Dv, v_row, BS, chunk, window,      \
-                     score_bias, sigmoid_weights, gate_per_head)
+                     score_bias, sigmoid_weights, gate_per_head, softcap)
 #define LIG_LAUNCH_ATT_H(T, VEC, NW)                    \
   if (hb == 4) LIG_LAUNCH_ATT(T, VEC, NW, 4);           \
   else if (hb == 2) LIG_LAUNCH_ATT(T, VEC, NW, 2);      \

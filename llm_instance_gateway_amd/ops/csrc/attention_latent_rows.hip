@@ -25,6 +25,9 @@
 // the (token, head) output row by one sigmoid (it commutes with whatever
 // linear map per head follows).
 //
+// window > 0 restricts a row at position p to keys j with p - j < window; a
+// tile's walk starts at the oldest key its first token sees.
+//
 // Grid = (ceil(max segment rows / 64), segments, splits); workgroups past a
 // segment's last row exit at once.  With splits > 1 (few rows, long
 // contexts) each z-slice walks an equal share of the tile's visible keys and
@@ -72,7 +75,7 @@ __global__ __launch_bounds__(256) void latent_attention_rows_kernel(
     const int* __restrict__ seg_start, const int* __restrict__ seg_len,
     const int* __restrict__ seg_ctx,     // tokens of the sequence after this step
     const int* __restrict__ block_tables, int max_blocks, float scale, int H,
-    int D, int Dv, int block_size, int nsplit,
+    int D, int Dv, int block_size, int window, int nsplit,
     float* __restrict__ partial) {  // [R * H, nsplit, Dv + 4] when nsplit > 1
   static_assert(DVP <= DKP, "values are a prefix of the key row");
   constexpr int DB = DVP / 16;
@@ -136,11 +139,14 @@ __global__ __launch_bounds__(256) void latent_attention_rows_kernel(
   const long last_rho = (rho0 + LR_ROWS < nrows ? rho0 + LR_ROWS : nrows) - 1;
   const int kv_end = ctx - n + (int)(last_rho / H) + 1;  // keys any row of the tile sees
 
-  int kv_lo = 0, kv_hi = kv_end;
+  // oldest key any row of the tile sees, and the one this lane's row sees
+  const int kv_first = window > 0 ? max(0, ctx - n + (int)(rho0 / H) - window + 1) : 0;
+  const int key_lo = window > 0 ? qpos - window + 1 : 0;
+  int kv_lo = kv_first, kv_hi = kv_end;
   if (nsplit > 1) {
-    const int nt = (kv_end + LR_KVBLK - 1) / LR_KVBLK;
+    const int nt = (kv_end - kv_first + LR_KVBLK - 1) / LR_KVBLK;
     const int per = (nt + nsplit - 1) / nsplit;
-    kv_lo = min(kv_end, z * per * LR_KVBLK);
+    kv_lo = min(kv_end, kv_first + z * per * LR_KVBLK);
     kv_hi = min(kv_end, kv_lo + per * LR_KVBLK);
   }
 
@@ -210,7 +216,7 @@ __global__ __launch_bounds__(256) void latent_attention_rows_kernel(
       for (int r = 0; r < 4; ++r) {
         const int key = kv0 + kt * 16 + lg * 4 + r;
         float v = acc_s[kt][r] * scale;
-        if (!row_valid || key > qpos) v = -INFINITY;
+        if (!row_valid || key > qpos || key < key_lo) v = -INFINITY;
         sc[kt * 4 + r] = v;
         rowmax = fmaxf(rowmax, v);
       }
@@ -389,7 +395,7 @@ extern "C" int lig_latent_attention_rows(
     const void* gate, long gate_stride,
     const int* seg_start, const int* seg_len, const int* seg_ctx,
     const int* block_tables, int max_blocks, float scale, int num_segs,
-    int max_seg_len, int H, int D, int Dv, int block_size, int nsplit,
+    int max_seg_len, int H, int D, int Dv, int block_size, int window, int nsplit,
     float* partial, hipStream_t stream) {
   if (D % 8 != 0 || Dv % 8 != 0 || D <= 0 || Dv <= 0 || Dv > D || D > 576 ||
       Dv > 512 || !aligned16(q) || !aligned16(cache) || H <= 0)
@@ -406,7 +412,7 @@ extern "C" int lig_latent_attention_rows(
                      (const uint16_t*)cache, sink,                             \
                      (const uint16_t*)gate, gate_stride, seg_start, seg_len,         \
                      seg_ctx, block_tables, max_blocks, scale, H, D, Dv,       \
-                     block_size, nsplit, partial)
+                     block_size, window, nsplit, partial)
   if (D <= 64 && Dv <= 64) LAUNCH_LR(64, 64);
   else if (D <= 128 && Dv <= 64) LAUNCH_LR(128, 64);
   else if (D <= 128) LAUNCH_LR(128, 128);

@@ -20,7 +20,8 @@
 // sink_h and its running sum at one (a key with that unscaled score and no
 // value).  chunk > 0 restricts a row at position p to keys j with
 // floor(j / chunk) == floor(p / chunk); window > 0 to keys j with
-// p - j < window.  sigmoid_weights replaces the softmax by unnormalised
+// p - j < window.  softcap > 0 bends every score, s <- softcap * tanh(s /
+// softcap).  sigmoid_weights replaces the softmax by unnormalised
 // weights sigmoid(score + score_bias[h]); gate_per_head reads one gate entry
 // per (row, head).  A value row is the first Dv entries of a cache row of v_row
 // entries, so a latent cache can pass its key rows as values.
@@ -29,6 +30,10 @@
 
 typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
 typedef float f32x4_t __attribute__((ext_vector_type(4)));
+
+// tanh through the hardware exponential; absolute error a few 1e-7, which a
+// soft cap scales by the cap
+LIG_DEVICE float pt_tanh(float x) { return 1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __expf(2.0f * x)); }
 
 #define PT_KVBLK 32
 #define PT_TQ 64
@@ -48,7 +53,7 @@ __global__ __launch_bounds__(256) void paged_attention_prefill_tiles_kernel(
     float temp_every, int temp_every_int, int num_q_heads, int num_kv_heads,
     int D, int Dv, int v_row, int block_size, int max_blocks, int chunk,
     int window, const float* __restrict__ score_bias, int sigmoid_weights,
-    int gate_per_head) {
+    int gate_per_head, float softcap) {
   constexpr int DB = DVP / 16;
   constexpr int KB = DKP / 32;
 
@@ -126,6 +131,7 @@ __global__ __launch_bounds__(256) void paged_attention_prefill_tiles_kernel(
     if (row_valid) key_lo = max(key_lo, qpos - window + 1);
   }
   const float sb = score_bias ? score_bias[h] : 0.f;
+  const float inv_cap = softcap > 0.f ? 1.0f / softcap : 0.f;
 
   for (int kv0 = kv_begin; kv0 < kv_end_tile; kv0 += PT_KVBLK) {
     // ---- staging: K rows [32][DKP], V transposed [DVP][32]; zero padding ----
@@ -188,6 +194,7 @@ __global__ __launch_bounds__(256) void paged_attention_prefill_tiles_kernel(
       for (int r = 0; r < 4; ++r) {
         const int key = kv0 + kt * 16 + lg * 4 + r;
         float v = acc_s[kt][r] * row_scale;
+        if (softcap > 0.f) v = softcap * pt_tanh(v * inv_cap);
         if (!row_valid || key > qpos || key >= ctx || key < key_lo) v = -INFINITY;
         sc[kt * 4 + r] = v;
         rowmax = fmaxf(rowmax, v);
@@ -293,7 +300,7 @@ extern "C" int lig_paged_attention_prefill_tiles(
     float temp_coef, float temp_every, int temp_every_int, int ntiles,
     int num_q_heads, int num_kv_heads, int D, int Dv, int v_row, int block_size,
     int max_blocks, int chunk, int window, const float* score_bias,
-    int sigmoid_weights, int gate_per_head, hipStream_t stream) {
+    int sigmoid_weights, int gate_per_head, float softcap, hipStream_t stream) {
   if (D % 8 != 0 || Dv % 8 != 0 || D > 128 || Dv > 128 || D <= 0 || Dv <= 0 ||
       v_row % 8 != 0 || v_row < Dv ||
       q_stride % 8 != 0 || !aligned16(q) || !aligned16(k_cache) ||
@@ -312,7 +319,7 @@ extern "C" int lig_paged_attention_prefill_tiles(
                      context_lens, block_tables, scale, temp_coef, temp_every, \
                      temp_every_int, num_q_heads, num_kv_heads, D, Dv, v_row, \
                      block_size, max_blocks, chunk, window, score_bias,       \
-                     sigmoid_weights, gate_per_head)
+                     sigmoid_weights, gate_per_head, softcap)
   const int dkp = D <= 32 ? 32 : (D <= 64 ? 64 : 128);
   const int dvp = Dv <= 32 ? 32 : (Dv <= 64 ? 64 : 128);
   if (dkp == 32 && dvp == 32) LAUNCH_PT(32, 32);

@@ -67,6 +67,14 @@ LIG_DEVICE float sigmoid_for<float>(float x) { return sigmoid_f32(x); }
 template <>
 LIG_DEVICE float sigmoid_for<bf16s>(float x) { return sigmoid_fast(x); }
 
+// The tanh form of gelu, 0.5 z (1 + tanh y) with y = sqrt(2/pi) (z + 0.044715
+// z^3), written as z * sigmoid(2 y): the same function, and no cancellation
+// where tanh is near -1.
+template <typename T>
+LIG_DEVICE float gelu_tanh_for(float z) {
+  return z * sigmoid_for<T>(1.59576912160573071176f * (z + 0.044715f * z * z * z));
+}
+
 // N consecutive elements (N = 1 or 4) <-> floats; N = 4 needs 8-byte (bf16)
 // or 16-byte (fp32) alignment.
 template <int N>

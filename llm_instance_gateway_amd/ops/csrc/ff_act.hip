@@ -55,8 +55,7 @@ __global__ void gelu_tanh_table_mul_kernel(T* __restrict__ out, const T* __restr
     ldn<N>(table + tokens[r] * table_stride + c, e);
 #pragma unroll
     for (int k = 0; k < N; ++k) {
-      const float a = v[k];
-      v[k] = 0.5f * a * (1.0f + tanhf(0.79788456080286535588f * (a + 0.044715f * a * a * a))) * e[k];
+      v[k] = gelu_tanh_for<T>(v[k]) * e[k];
     }
     stn<N>(out + i, v);
   }

@@ -11,6 +11,8 @@
 //   norm         : out      = norm(residual) * w                (f32 -> T)
 //   post_add_pre : residual += norm(y) * w_post;                (T  -> f32)
 //                  out = norm(residual) * w_pre                 (f32 -> T)
+//                  (w_pre null: out = residual rounded to T, for stacks
+//                  whose sub-layers read the residual itself)
 // The last one fuses a sub-layer's output norm, the residual add and the
 // next sub-layer's input norm: one pass over y and the residual instead of
 // three kernels.
@@ -100,6 +102,14 @@ __global__ void post_add_pre_norm_vec_kernel(T* __restrict__ out,
     }
   }
   if (out == nullptr) return;  // uniform across the block
+  if (w_pre == nullptr) {      // the next sub-layer reads the sum itself
+#pragma unroll
+    for (int k = 0; k < VPT; ++k) {
+      const int idx = threadIdx.x + k * blockDim.x;
+      if (idx < nvec) st8(out + base + idx * 8, v[k]);
+    }
+    return;
+  }
   ss2 = block_reduce_sum(ss2, lds);
   const float inv_r = 1.0f / sqrtf(ss2 / (float)P + eps);
 #pragma unroll
@@ -166,6 +176,10 @@ __global__ void post_add_pre_norm_scalar_kernel(T* __restrict__ out,
     ss2 += r * r;
   }
   if (out == nullptr) return;  // uniform across the block
+  if (w_pre == nullptr) {      // the next sub-layer reads the sum itself
+    for (int i = threadIdx.x; i < P; i += blockDim.x) st(out + base + i, res[i]);
+    return;
+  }
   ss2 = block_reduce_sum(ss2, lds);
   const float inv_r = 1.0f / sqrtf(ss2 / (float)P + eps);
   const T* wn = w_pre + (size_t)g * P;
@@ -257,7 +271,8 @@ void lig_group_norm(void* out, const float* residual, const void* w, float eps,
                                      (const bf16s*)w, eps, rows, H, groups, s);
 }
 
-// out may be null: then only the residual update is done.
+// out may be null: then only the residual update is done.  w_pre may be null:
+// then out is the new residual rounded to the storage type.
 void lig_post_add_pre_norm(void* out, float* residual, const void* y,
                            const void* w_post, const void* w_pre, float eps,
                            int rows, int H, int groups, int is_f32,

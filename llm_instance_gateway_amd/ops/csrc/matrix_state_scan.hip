@@ -13,6 +13,11 @@
 //       S_t = exp(f + m_{t-1} - m_t) S_{t-1} + exp(i - m_t) k_t v_t^T
 //       n_t likewise with k_t alone
 //       o_t = S_t^T q_t / (max(|n_t . q_t|, exp(-m_t)) + 1e-6)
+//   delta form (a decay g and a write strength b per head and token; k and q
+//   are unit vectors, several value heads may share a q/k head):
+//       S  <- g S;  u = b (v - S^T k);  S <- S + k u^T
+//       o_t = S^T q_t
+//       g = exp(-exp(rate) softplus(z + bias)),  b = sigmoid(z_b)
 //   optional on q and k as they are read: silu (also on v), a rotate-half
 //   rotation by tabulated cosines and sines, a constant factor each.
 //
@@ -39,8 +44,12 @@
 // (ops.matrix_state_width mirrors this).
 // A segment that starts its sequence ignores what the slot held.
 //
-// Long bf16 portions of the constant-decay and gated forms are handed to the
-// chunked MFMA kernel, which reads and writes the same state rows.
+// The delta form's dot of k with the state is one more sum over the lanes of a
+// column ahead of the update.  The unit norms stay outside the vectors: with
+// k = kr / |kr| and raw kr in LDS, S^T k and k u^T take the factor as a scalar.
+//
+// Long bf16 portions of the constant-decay, gated and delta forms are handed
+// to the chunked MFMA kernels, which read and write the same state rows.
 
 #include "matrix_state.h"
 
@@ -89,7 +98,7 @@ LIG_DEVICE float ms_prep(const T* __restrict__ x, int i, const float* __restrict
 template <typename T, int MS_SPLIT, int KPT, int FORM, int MAXT>
 __global__ __launch_bounds__(MAXT) void matrix_state_scan_kernel(const MsArgs A) {
   extern __shared__ __align__(16) float sm[];
-  constexpr bool BONUS = FORM == MS_BONUS, GATED = FORM == MS_GATED;
+  constexpr bool BONUS = FORM == MS_BONUS, GATED = FORM == MS_GATED, DELTA = FORM == MS_DELTA;
   constexpr int Dp = MS_SPLIT * KPT;
   const int H = A.H, D = A.D, Dv = A.Dv, TT = A.TT;
   const int CBw = GATED ? A.CB + 1 : A.CB;  // columns that own state
@@ -97,10 +106,11 @@ __global__ __launch_bounds__(MAXT) void matrix_state_scan_kernel(const MsArgs A)
   float* k_s = q_s + TT * Dp;      // [TT][Dp]
   float* w_s = k_s + TT * Dp;      // [TT][Dp] (BONUS only)
   float* v_s = BONUS ? w_s + TT * Dp : w_s;  // [TT][CBw]
-  float* o_s = v_s + TT * CBw;     // [TT][CBw] (GATED only), then
-  float* a_s = o_s + TT * CBw;     // [TT] kept share of the state,
-  float* b_s = a_s + TT;           // [TT] weight of the new key,
-  float* e_s = b_s + TT;           // [TT] exp(-m)
+  float* o_s = v_s + TT * CBw;     // [TT][CBw] (GATED), then
+  float* a_s = GATED ? o_s + TT * CBw : o_s;  // [TT] kept share of the state,
+  float* b_s = a_s + TT;           // [TT] weight of the new key (DELTA: write strength),
+  float* e_s = b_s + TT;           // [TT] exp(-m); DELTA: 1 / |k|,
+  float* f_s = e_s + TT;           // [TT] DELTA: q_scale / |q|
 
   const int seg = blockIdx.x, h = blockIdx.y, blk = blockIdx.z;
   const int n = A.seg_len[seg];
@@ -111,8 +121,9 @@ __global__ __launch_bounds__(MAXT) void matrix_state_scan_kernel(const MsArgs A)
   const bool owner = j < CBw;
   const int nthr = CBw * MS_SPLIT;  // threads that own state
   const int c0 = blk * A.CB, ncol = min(A.CB, Dv - c0);
-  const T* q = (const T*)A.q + h * D;
-  const T* k = (const T*)A.k + h * D;
+  const int hk = DELTA ? h / A.rep : h;
+  const T* q = (const T*)A.q + hk * D;
+  const T* k = (const T*)A.k + hk * D;
   const T* v = (const T*)A.v + h * Dv + c0;
 
   float S[KPT], U[KPT];
@@ -140,7 +151,8 @@ __global__ __launch_bounds__(MAXT) void matrix_state_scan_kernel(const MsArgs A)
       float qv = 0.f, kv = 0.f, wv = 0.f;
       if (i < D) {
         const float* cs = A.cs + r * 2 * A.nf;
-        qv = ms_prep(q + r * A.q_stride, i, cs, A.nf, A.q_scale, A.act_silu);
+        // (delta form: the scale joins the unit norm's factor)
+        qv = ms_prep(q + r * A.q_stride, i, cs, A.nf, DELTA ? 1.0f : A.q_scale, A.act_silu);
         kv = ms_prep(k + r * A.k_stride, i, cs, A.nf, A.k_scale, A.act_silu);
         if (BONUS) wv = expf(-expf(A.decay_pre[r * (long)(H * D) + h * D + i]));
       }
@@ -157,6 +169,11 @@ __global__ __launch_bounds__(MAXT) void matrix_state_scan_kernel(const MsArgs A)
         if (A.act_silu) vv = vv * sigmoid_f32(vv);
       }
       v_s[e] = vv;
+    }
+    if (DELTA && tid < nt_tok) {
+      const long r = (long)(r0 + t0 + tid) * A.gate_stride + h;
+      a_s[tid] = expf(ms_log_decay(A.gate_f[r], A.bias_i[h], A.bias_f[h]));
+      b_s[tid] = sigmoid_f32(A.gate_i[r]);
     }
     if (GATED && tid < WAVE_SIZE) {
       // lane t: gates of token t, prefix sum of the log forget gates, prefix
@@ -191,6 +208,23 @@ __global__ __launch_bounds__(MAXT) void matrix_state_scan_kernel(const MsArgs A)
       m_run = __shfl(m, nt_tok - 1, WAVE_SIZE);
     }
     __syncthreads();
+    if (DELTA) {
+      // lengths of the staged q and k, a wave per token
+      for (int t = tid / WAVE_SIZE; t < nt_tok; t += nt / WAVE_SIZE) {
+        float sq = 0.f, sk = 0.f;
+        for (int i = tid % WAVE_SIZE; i < Dp; i += WAVE_SIZE) {
+          sq += q_s[t * Dp + i] * q_s[t * Dp + i];
+          sk += k_s[t * Dp + i] * k_s[t * Dp + i];
+        }
+        sq = wave_reduce_sum(sq);
+        sk = wave_reduce_sum(sk);
+        if (tid % WAVE_SIZE == 0) {
+          e_s[t] = 1.0f / sqrtf(sk + A.unit_eps);
+          f_s[t] = A.q_scale / sqrtf(sq + A.unit_eps);
+        }
+      }
+      __syncthreads();
+    }
     // every wave of the workgroup walks the tile (idle lanes of the last
     // wave take part in the lane permutes with zeros)
     // one token: read its q, k, decay and v from LDS, output, state update
@@ -202,6 +236,35 @@ __global__ __launch_bounds__(MAXT) void matrix_state_scan_kernel(const MsArgs A)
       const float* kt = k_s + t * Dp + s * KPT;
       const float* wt = w_s + t * Dp + s * KPT;
       float o = 0.f;
+      if (DELTA) {
+        const float g = a_s[t], ik = e_s[t];
+        float held = 0.f;
+#pragma unroll
+        for (int i4 = 0; i4 < KPT; i4 += 4) {
+          const f32x4 k4 = *reinterpret_cast<const f32x4*>(kt + i4);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            S[i4 + e] *= g;
+            held += k4[e] * S[i4 + e];
+          }
+        }
+        held = split_sum<MS_SPLIT>(held);
+        const float u = b_s[t] * (vj - held * ik) * ik;
+#pragma unroll
+        for (int i4 = 0; i4 < KPT; i4 += 4) {
+          const f32x4 k4 = *reinterpret_cast<const f32x4*>(kt + i4);
+          const f32x4 q4 = *reinterpret_cast<const f32x4*>(qt + i4);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            S[i4 + e] += k4[e] * u;
+            o += q4[e] * S[i4 + e];
+          }
+        }
+        o = split_sum<MS_SPLIT>(o) * f_s[t];
+        if (owner && s == 0 && j < ncol)
+          A.out[(long)(r0 + t0 + t) * (H * Dv) + h * Dv + c0 + j] = o;
+        return;
+      }
 #pragma unroll
       for (int i4 = 0; i4 < KPT; i4 += 4) {
         const f32x4 k4 = *reinterpret_cast<const f32x4*>(kt + i4);
@@ -317,7 +380,7 @@ extern "C" int lig_matrix_state_scan(
   MsArgs a{out, q, k, v, q_stride, k_stride, v_stride, decay_pre, head_decay, bonus,
                  gate_i, gate_f, gate_stride, bias_i, bias_f, gate_cap, cs, nf, q_scale,
                  k_scale, state, state_stride, seg_start, seg_len, seg_slot, seg_fresh,
-                 H, D, Dv, CB, NB, TT, act_silu, split, kpt, 1, INT_MAX};
+                 H, D, Dv, CB, NB, TT, act_silu, split, kpt, 1, INT_MAX, 1, 0.f};
   const dim3 grid(S, H, NB);
   if (max_seg_len >= MS_CHUNK_MIN && !is_f32 && !act_silu && form != MS_BONUS &&
       ms_chunks_served(a, form)) {
@@ -339,5 +402,47 @@ extern "C" int lig_matrix_state_scan(
     LIG_MS_FORM(bf16s);
   }
 #undef LIG_MS_FORM
+  return 0;
+}
+
+// The delta form.  gate_b: write-strength logits, gate_a: decay logits (fp32
+// [R, H] views with one row stride); log_rate, bias: fp32 [H].  q and k hold
+// KH heads, value head h reads head h / (H / KH).  scratch (chunked portions,
+// may be null: everything is walked) holds lig_gated_delta_scratch bytes.
+// Segments lie in row order.  Returns 0 when launched, 1 when a head is wider
+// than the kernel holds or the heads do not divide.
+extern "C" int lig_gated_delta_scan(
+    float* out, const void* q, long q_stride, const void* k, long k_stride, const void* v,
+    long v_stride, const float* gate_b, const float* gate_a, long gate_stride,
+    const float* log_rate, const float* bias, float q_scale, float unit_eps, float* state,
+    long state_stride, const int* seg_start, const int* seg_len, const int* seg_slot,
+    const int* seg_fresh, int S, int H, int KH, int D, int Dv, int max_seg_len, void* scratch,
+    int is_f32, hipStream_t stream) {
+  int split = 4, kpt = 0;
+  if (D > 0) ms_shape(D, &split, &kpt);
+  if (kpt == 0 || Dv <= 0 || KH <= 0 || H % KH != 0) return 1;
+  const int CB = Dv < MS_COLS ? Dv : MS_COLS;
+  const int NB = (Dv + CB - 1) / CB;
+  if (H > 65535 || NB > 65535) return 1;
+  if (S <= 0) return 0;
+  const int Dp = kpt * split;
+  const int per_tok = 2 * Dp + CB + 4;
+  const int TT = per_tok * 32 * 4 <= 40 * 1024 ? 32 : (per_tok * 16 * 4 <= 48 * 1024 ? 16 : 8);
+  const size_t smem = (size_t)per_tok * TT * sizeof(float);
+  const int threads = ((CB * split + WAVE_SIZE - 1) / WAVE_SIZE) * WAVE_SIZE;
+  MsArgs a{out, q, k, v, q_stride, k_stride, v_stride, nullptr, nullptr, nullptr,
+           gate_b, gate_a, gate_stride, log_rate, bias, 1.0f, nullptr, 0, q_scale,
+           1.0f, state, state_stride, seg_start, seg_len, seg_slot, seg_fresh,
+           H, D, Dv, CB, NB, TT, 0, split, kpt, 1, INT_MAX, H / KH, unit_eps};
+  const dim3 grid(S, H, NB);
+  if (max_seg_len >= MS_CHUNK_MIN && !is_f32 && scratch != nullptr && ms_delta_chunks_served(a)) {
+    a.len_min = MS_CHUNK_MIN;
+    ms_delta_chunks_launch(a, S, max_seg_len, scratch, stream);
+    if (S == 1) return 0;
+    a.len_min = 1;
+    a.len_max = MS_CHUNK_MIN - 1;
+  }
+  if (is_f32) ms_dispatch<float, MS_DELTA>(a, split, kpt, grid, threads, smem, stream);
+  else ms_dispatch<bf16s, MS_DELTA>(a, split, kpt, grid, threads, smem, stream);
   return 0;
 }

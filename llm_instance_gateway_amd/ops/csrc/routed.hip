@@ -25,6 +25,7 @@
 //   0: relu(gate) * up
 //   1: g = min(gate, limit), u = clamp(up, -limit, limit),
 //      g * sigmoid(alpha * g) * (u + 1)
+//   2: gelu_tanh(gate) * up, the tanh form of gelu
 
 #include "elem_types.h"
 
@@ -190,6 +191,8 @@ __global__ void glu_act_kernel(T* __restrict__ out, const T* __restrict__ x, int
     for (int k = 0; k < N; ++k) {
       if (KIND == 0) {
         g[k] = fmaxf(g[k], 0.f) * u[k];
+      } else if (KIND == 2) {
+        g[k] = gelu_tanh_for<T>(g[k]) * u[k];
       } else {
         const float gg = fminf(g[k], limit);
         const float uu = fminf(fmaxf(u[k], -limit), limit);
@@ -260,7 +263,7 @@ void lig_glu_act(void* out, const void* x, long rows, int F, int kind, float lim
   hipLaunchKernelGGL((glu_act_kernel<T, N, K>), dim3(grid), dim3(256), 0, s,    \
                      (T*)out, (const T*)x, F, n, limit, alpha)
 #define LIG_GA_K(T, N) \
-  if (kind == 0) LIG_GA(T, N, 0); else LIG_GA(T, N, 1)
+  if (kind == 0) LIG_GA(T, N, 0); else if (kind == 1) LIG_GA(T, N, 1); else LIG_GA(T, N, 2)
   if (is_f32) {
     if (v4) { LIG_GA_K(float, 4); } else { LIG_GA_K(float, 1); }
   } else {

@@ -2,7 +2,7 @@
 minGRU scan, general-size paged attention, shift norms, latent attention,
 sum+norm residual step, q/k/v prep, head-mixed attention, matrix-state scan,
 multi-stream residual step, grouped router and routed combine, layer norms,
-fp32 projections onto a few columns).
+fp32 projections onto a few columns, short convolutions, gated delta rule).
 
 These kernels expose a plain C ABI and need no torch headers, so they are
 compiled by direct ``hipcc`` calls (side by side, without the minutes the
@@ -37,7 +37,7 @@ SOURCES = [
     "attention_prefill_tiles.hip", "shift_norm.hip", "latent_attention.hip", "ff_act.hip",
     "attention_latent_rows.hip", "post_norm.hip", "qkv_prep.hip", "attention_mixed_heads.hip",
     "matrix_state_scan.hip", "matrix_state_chunks.hip", "attention_mixed_heads_tiles.hip", "hyper_streams.hip",
-    "routed.hip", "layer_norm.hip", "small_projection.hip",
+    "routed.hip", "layer_norm.hip", "small_projection.hip", "short_conv.hip", "matrix_state_delta.hip",
 ]
 SO_PATH = PKG / "_hybrid.so"
 
@@ -94,7 +94,7 @@ def _declare(lib: ctypes.CDLL) -> None:
         "lig_mingru_scan": [p, p, p, p, l, p, p, p, p, p, p, i, i, i, i, p],
         "lig_paged_attention_general": [
             p, p, l, p, p, p, i, p, p, p, l, p, f, f, f, i, i, i, i, i, i, i, i, i,
-            i, p, i, i, i, p,
+            i, p, i, i, f, i, p,
         ],
         "lig_offset_norm_shift": [p, p, p, p, p, p, p, p, p, p, p, p, p, p, p, f, i, i, i, p],
         "lig_offset_rms_norm": [p, p, p, f, i, i, i, p],
@@ -129,7 +129,7 @@ def _declare(lib: ctypes.CDLL) -> None:
     pt = lib.lig_paged_attention_prefill_tiles
     pt.argtypes = [
         p, p, l, p, p, p, l, p, p, p, p, p, p, f, f, f, i, i, i, i, i, i, i, i, i, i,
-        i, p, i, i, p,
+        i, p, i, i, f, p,
     ]
     pt.restype = ctypes.c_int
     hs = lib.lig_hyper_step
@@ -157,8 +157,19 @@ def _declare(lib: ctypes.CDLL) -> None:
     ]
     ms.restype = ctypes.c_int
     lr = lib.lig_latent_attention_rows
-    lr.argtypes = [p, p, p, p, p, l, p, p, p, p, i, f, i, i, i, i, i, i, i, p, p]
+    lr.argtypes = [p, p, p, p, p, l, p, p, p, p, i, f, i, i, i, i, i, i, i, i, p, p]
     lr.restype = ctypes.c_int
+    sc = lib.lig_short_conv_silu
+    sc.argtypes = [p, p, l, p, p, l, p, p, p, p, i, i, i, i, i, p]
+    sc.restype = ctypes.c_int
+    gd = lib.lig_gated_delta_scan
+    gd.argtypes = [
+        p, p, l, p, l, p, l, p, p, l, p, p, f, f, p, l, p, p, p, p, i, i, i, i, i, i, p, i, p,
+    ]
+    gd.restype = ctypes.c_int
+    gs = lib.lig_gated_delta_scratch
+    gs.argtypes = [i, i, i]
+    gs.restype = l
 
 
 def lib() -> ctypes.CDLL:

@@ -292,7 +292,7 @@ def paged_attention_general(
     q, k_cache, v_cache, block_tables, tok_seq, positions, scale: float,
     num_heads: int, gate=None, temp_coef: float = 0.0, temp_every: float = 1.0,
     sink=None, chunk: int = 0, window: int = 0, score_bias=None,
-    weights: str = "softmax", gate_per_head: bool = False,
+    weights: str = "softmax", gate_per_head: bool = False, softcap: float = 0.0,
 ):
     """q [R, H*D] (may be a strided view); token r belongs to sequence row
     tok_seq[r] of block_tables (-1: padding row) and sees keys 0..positions[r].
@@ -302,7 +302,7 @@ def paged_attention_general(
     only if floor(j / chunk) == floor(position / chunk); window > 0 hides
     keys with position - j >= window.  weights "sigmoid": unnormalised
     sigmoid(score + score_bias[h]) per visible key.  gate_per_head: gate
-    [R, H]."""
+    [R, H].  softcap > 0: score <- softcap * tanh(score / softcap)."""
     R = q.shape[0]
     nb, G, bs, D = k_cache.shape
     Dv = v_cache.shape[-1]
@@ -331,6 +331,8 @@ def paged_attention_general(
             vf = v.repeat_interleave(H // G, dim=1).permute(1, 0, 2)
             qf = q[r:e].float().reshape(e - r, H, D).permute(1, 0, 2)  # [H, n, D]
             sc = torch.bmm(qf, kf.transpose(1, 2)) * (scale * tau[r:e])[None, :, None]
+            if softcap > 0.0:
+                sc = softcap * torch.tanh(sc / softcap)
             keyp = torch.arange(L, device=q.device)[None, :]
             mask = keyp > positions[r:e, None]
             if chunk > 0:
@@ -411,11 +413,22 @@ def offset_norm_shift(
     return hm.to(out_dtype), hf
 
 
-def rotary_inv_freq(base: float, dims: int, device=None, divide: float = 1.0) -> torch.Tensor:
+def rotary_inv_freq(
+    base: float, dims: int, device=None, divide: float = 1.0, scaling=None
+) -> torch.Tensor:
     """f_i = base^(-2i/dims) / divide, i < dims/2, evaluated in float64, stored
-    fp32 (divide > 1 is linear position scaling)."""
+    fp32 (divide > 1 is linear position scaling).  `scaling` {factor, low,
+    high, original} then works by bands of the wavelength l = 2 pi / f: kept
+    where l < original / high, divided by factor where l > original / low, a
+    linear ramp in original / l between."""
     i = torch.arange(dims // 2, dtype=torch.float64)
     f = torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / dims) / float(divide)
+    if scaling:
+        factor, low, high, original = (float(scaling[k]) for k in ("factor", "low", "high", "original"))
+        wave = 2.0 * math.pi / f
+        s = (original / wave - low) / (high - low)
+        ramp = (1.0 - s) * f / factor + s * f
+        f = torch.where(wave > original / low, f / factor, torch.where(wave < original / high, f, ramp))
     return f.float().to(device)
 
 
@@ -659,6 +672,58 @@ def matrix_state_scan(
     return out.view(R, heads * vdim)
 
 
+def short_conv_silu(x, w, state, seg_start, seg_len, seg_slot, seg_fresh):
+    R, C = x.shape
+    taps = w.shape[0]
+    out = torch.zeros(R, C, dtype=x.dtype, device=x.device)
+    for s0, n, slot, fresh in zip(
+        seg_start.tolist(), seg_len.tolist(), seg_slot.tolist(), seg_fresh.tolist()
+    ):
+        if n <= 0:
+            continue
+        old = state[slot].view(taps - 1, C)
+        ext = torch.cat([torch.zeros_like(old) if fresh else old, x[s0 : s0 + n].float()])
+        y = sum(w[j].float() * ext[j : j + n] for j in range(taps))
+        out[s0 : s0 + n] = torch.nn.functional.silu(y).to(x.dtype)
+        state[slot] = ext[n:].reshape(-1)
+    return out
+
+
+def gated_delta_scan(
+    q, k, v, b, a, log_rate, bias, state, seg_start, seg_len, seg_slot, seg_fresh, heads: int,
+    kv_heads: int, dim: int, vdim: int, q_scale: float, unit_eps: float,
+):
+    R = q.shape[0]
+
+    def unit(t):
+        t = t.float().reshape(R, kv_heads, dim)
+        t = t / torch.sqrt(t.pow(2).sum(-1, keepdim=True) + unit_eps)
+        return t.repeat_interleave(heads // kv_heads, dim=1)
+
+    qf, kf, vf = unit(q) * q_scale, unit(k), v.float().reshape(R, heads, vdim)
+    g = torch.exp(-torch.exp(log_rate.float()) * torch.nn.functional.softplus(a + bias, threshold=1e9))
+    beta = torch.sigmoid(b)
+    out = torch.zeros(R, heads, vdim, dtype=torch.float32, device=q.device)
+    nS = heads * dim * vdim
+    for s0, n, slot, fresh in zip(
+        seg_start.tolist(), seg_len.tolist(), seg_slot.tolist(), seg_fresh.tolist()
+    ):
+        if n <= 0:
+            continue
+        S = (
+            torch.zeros(heads, dim, vdim, dtype=torch.float32, device=q.device)
+            if fresh else state[slot, :nS].view(heads, dim, vdim).clone()
+        )
+        for t in range(s0, s0 + n):
+            S = g[t][:, None, None] * S
+            held = torch.einsum("hd,hde->he", kf[t], S)
+            u = beta[t][:, None] * (vf[t] - held)
+            S = S + kf[t][:, :, None] * u[:, None, :]
+            out[t] = torch.einsum("hd,hde->he", qf[t], S)
+        state[slot, :nS] = S.reshape(-1)
+    return out.view(R, heads * vdim)
+
+
 def _rotate_halves_table(v: torch.Tensor, cs: torch.Tensor) -> torch.Tensor:
     """v [R, H, D] fp32: entries i and i + n of every head turn by the angle
     whose cosine and sine are cs[r, i] and cs[r, n + i]."""
@@ -782,6 +847,8 @@ def glu_act(x, kind: str, limit: float, alpha: float):
     g, u = x[:, :F_].float(), x[:, F_:].float()
     if kind == "relu":
         return (torch.relu(g) * u).to(x.dtype)
+    if kind == "gelu_tanh":
+        return (torch.nn.functional.gelu(g, approximate="tanh") * u).to(x.dtype)
     g = g.clamp(max=limit)
     u = u.clamp(min=-limit, max=limit)
     return (g * torch.sigmoid(alpha * g) * (u + 1.0)).to(x.dtype)

@@ -13,7 +13,7 @@ import torch
 
 from llm_instance_gateway_amd import ops
 from llm_instance_gateway_amd.models.hybrid_blocks import (
-    GatedReluMLP, GroupRoutedExpertsMLP, expert_dispatch_plan,
+    GatedMLP, GroupRoutedExpertsMLP, expert_dispatch_plan,
 )
 
 import vemenex_oracle as O
@@ -325,7 +325,7 @@ def test_gated_relu_mlp(device, dtype):
     H, ff, T = 24, 17, 6
     W = {"gate": rnd(g, ff, H, s=H ** -0.5).to(dtype), "up": rnd(g, ff, H, s=H ** -0.5).to(dtype),
          "down": rnd(g, H, ff, s=ff ** -0.5).to(dtype)}
-    mod = GatedReluMLP(H, ff, device=device, dtype=dtype)
+    mod = GatedMLP(H, ff, "relu", device=device, dtype=dtype)
     mod.load(lambda n: W[n].to(device), "")
     h = rnd(g, T, H).to(dtype)
     want = O.dense_ff(h.double().numpy(), {k: v.double().numpy() for k, v in W.items()})
