@@ -158,7 +158,27 @@ def main() -> None:
         "PARTS = engine, kernels or both (benchmarks/bench_recurrent.py)",
     )
     ap.add_argument("--recurrent-sizes", default="s,m")
+    ap.add_argument(
+        "--delta",
+        nargs="?",
+        const="engine,kernels",
+        default="",
+        metavar="PARTS",
+        help="instead of the serving workload: Daberax (gated delta rule, "
+        "windowed latent and soft-capped attention, norms on the sub-layers' "
+        "outputs) beside Garesun and Potatar at equal size, and its kernels "
+        "beside their counterparts against the roofline; PARTS = engine, "
+        "kernels or both (benchmarks/bench_delta.py)",
+    )
+    ap.add_argument("--delta-sizes", default="s,m")
     args = ap.parse_args()
+
+    if args.delta:
+        sys.path.insert(0, os.path.join(os.path.dirname(os.path.abspath(__file__)), "benchmarks"))
+        import bench_delta
+
+        bench_delta.main(["--part", args.delta, "--sizes", args.delta_sizes])
+        return
 
     if args.recurrent:
         sys.path.insert(0, os.path.join(os.path.dirname(os.path.abspath(__file__)), "benchmarks"))
