@@ -19,6 +19,7 @@ Prefill / mixed steps stay eager (their shapes vary too much to bucket).
 
 from __future__ import annotations
 
+import gc
 import logging
 from typing import Dict, List, Optional
 
@@ -205,16 +206,28 @@ class DecodeGraphRunner:
                 self._forward(B)
         torch.cuda.current_stream(self.device).wait_stream(s)
         torch.cuda.synchronize(self.device)
-        for B in self.sizes:
-            g = torch.cuda.CUDAGraph()
-            if self._pool is None:
-                with torch.cuda.graph(g):
-                    self.logits[B] = self._forward(B)
-                self._pool = g.pool()
-            else:
-                with torch.cuda.graph(g, pool=self._pool):
-                    self.logits[B] = self._forward(B)
-            self.graphs[B] = g
+        # Graphs of an engine that is no longer referenced sit in reference
+        # cycles; if the collector freed one of them in the middle of a
+        # capture, its destructor would call into the runtime, which is not
+        # permitted then and ends the process.  Collect now, and hold the
+        # collector off until the captures are done.
+        gc.collect()
+        gc_was_on = gc.isenabled()
+        gc.disable()
+        try:
+            for B in self.sizes:
+                g = torch.cuda.CUDAGraph()
+                if self._pool is None:
+                    with torch.cuda.graph(g):
+                        self.logits[B] = self._forward(B)
+                    self._pool = g.pool()
+                else:
+                    with torch.cuda.graph(g, pool=self._pool):
+                        self.logits[B] = self._forward(B)
+                self.graphs[B] = g
+        finally:
+            if gc_was_on:
+                gc.enable()
         torch.cuda.synchronize(self.device)
         log.info("captured %d decode graphs (lora=%s)", len(self.graphs), with_lora)
 

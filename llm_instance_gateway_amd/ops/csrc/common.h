@@ -24,15 +24,9 @@ LIG_DEVICE float bf16_to_f32(uint16_t h) {
   return v.f;
 }
 
+// round-to-nearest-even, one hardware conversion
 LIG_DEVICE uint16_t f32_to_bf16(float f) {
-  union {
-    float f;
-    uint32_t u;
-  } v;
-  v.f = f;
-  // round-to-nearest-even
-  uint32_t rounding_bias = ((v.u >> 16) & 1u) + 0x7FFFu;
-  return static_cast<uint16_t>((v.u + rounding_bias) >> 16);
+  return __builtin_bit_cast(uint16_t, static_cast<__bf16>(f));
 }
 
 // 8 bf16 = 16 B: the unit of a fully-coalesced per-lane load (guide §2:

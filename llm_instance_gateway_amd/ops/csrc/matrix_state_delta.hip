@@ -65,10 +65,13 @@ template <int DP>
 __global__ __launch_bounds__(DI_THREADS) void delta_chunk_inverse_kernel(
     const MsArgs A, DeltaChunk* __restrict__ scratch) {
   constexpr int KB = DP / 32;
-  __shared__ float a_s[MC_T][DI_ROW];
-  __shared__ float t_s[MC_T][DI_ROW];
+  // One square holds both triangles in 16 x 16 blocks: the system's block (i,
+  // j) at its own place, the inverse's block (i, j) at place (j, i), each in
+  // row order; a diagonal block of the inverse replaces the system's.
+  __shared__ __align__(16) float a_s[MC_T][DI_ROW];
   __shared__ double g_s[MC_T];
-  __shared__ float b_s[MC_T], ik_s[MC_T];
+  __shared__ __align__(16) float b_s[MC_T];
+  __shared__ float ik_s[MC_T];
 
   const int seg = blockIdx.y, h = blockIdx.z;
   const int n = A.seg_len[seg];
@@ -151,7 +154,7 @@ __global__ __launch_bounds__(DI_THREADS) void delta_chunk_inverse_kernel(
     }
     if (lg == 0) {
 #pragma unroll
-      for (int i = 0; i < 16; ++i) t_s[b + i][b + li] = x[i];
+      for (int i = 0; i < 16; ++i) a_s[b + i][b + li] = x[i];
     }
   }
   __syncthreads();
@@ -164,14 +167,14 @@ __global__ __launch_bounds__(DI_THREADS) void delta_chunk_inverse_kernel(
       for (int m = bj; m < bi; m += 16) {
 #pragma unroll
         for (int e = 0; e < 16; e += 4)
-          x = __builtin_amdgcn_mfma_f32_16x16x4f32(a_s[bi + li][m + e + lg], t_s[m + e + lg][bj + li],
+          x = __builtin_amdgcn_mfma_f32_16x16x4f32(a_s[bi + li][m + e + lg], a_s[bj + e + lg][m + li],
                                                    x, 0, 0, 0);
       }
 #pragma unroll
       for (int r = 0; r < 4; ++r)  // x's rows lg * 4 + r are this lane's share of the contraction
-        y = __builtin_amdgcn_mfma_f32_16x16x4f32(t_s[bi + li][bi + lg * 4 + r], x[r], y, 0, 0, 0);
+        y = __builtin_amdgcn_mfma_f32_16x16x4f32(a_s[bi + li][bi + lg * 4 + r], x[r], y, 0, 0, 0);
 #pragma unroll
-      for (int r = 0; r < 4; ++r) t_s[bi + lg * 4 + r][bj + li] = -y[r];
+      for (int r = 0; r < 4; ++r) a_s[bj + lg * 4 + r][bi + li] = -y[r];
     }
     __syncthreads();
   }
@@ -179,19 +182,18 @@ __global__ __launch_bounds__(DI_THREADS) void delta_chunk_inverse_kernel(
   {
     const int t = tid >> 2, s0 = (tid & 3) * 16;
     if (s0 <= t) {
+      const float* src = &a_s[s0 + (t & 15)][t & ~15];  // row t of block (t / 16, s0 / 16)
 #pragma unroll
       for (int half = 0; half < 2; ++half) {
-        u16x8 hi, lo;
+        u32x4 hi, lo;
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          const int s = s0 + half * 8 + e;
-          uint16_t a, b;
-          mc_split(t_s[t][s] * b_s[s], a, b);
-          hi[e] = a;
-          lo[e] = b;
+        for (int e = 0; e < 2; ++e) {
+          const int s = half * 8 + e * 4;
+          mc_split4(*reinterpret_cast<const f32x4*>(src + s) *
+                        *reinterpret_cast<const f32x4*>(&b_s[s0 + s]), e, hi, lo);
         }
-        *reinterpret_cast<u16x8*>(&out->t_hi[t][s0 + half * 8]) = hi;
-        *reinterpret_cast<u16x8*>(&out->t_lo[t][s0 + half * 8]) = lo;
+        *reinterpret_cast<u32x4*>(&out->t_hi[t][s0 + half * 8]) = hi;
+        *reinterpret_cast<u32x4*>(&out->t_lo[t][s0 + half * 8]) = lo;
       }
     }
   }
@@ -211,22 +213,24 @@ __global__ __launch_bounds__(DI_THREADS) void delta_chunk_inverse_kernel(
 template <int DP, int NW>
 __global__ __launch_bounds__(NW * WAVE_SIZE) void delta_chunk_scan_kernel(
     const MsArgs A, const DeltaChunk* __restrict__ scratch) {
-  constexpr int KB = DP / 32, DT = DP / 16, DROW = DP + 8;
+  // LDS rows advance by 2 banks (mod 32), so that the 8-byte operand reads of
+  // 16 rows spread over all of them
+  constexpr int KB = DP / 32, DT = DP / 16, DROW = DP + 4, TROW = MC_T + 4;
   constexpr int CC = DP / 8;                  // 16-byte chunks of a q or k row
   constexpr int NCH = (CC + NW - 1) / NW;     // of them per thread
   constexpr int NT = 2 * MC_T * MC_T / 8 / (NW * WAVE_SIZE);  // inverse chunks per thread
   struct Shared {
     uint16_t q[MC_T][DROW];
     uint16_t k[MC_T][DROW];
-    uint16_t kt[DP][MC_TP];
-    uint16_t t[2][MC_T][MC_TP];
-    uint16_t p[2][MC_T][MC_TP];
+    uint16_t kt[DP][TROW];
+    uint16_t t[2][MC_T][TROW];
+    uint16_t p[2][MC_T][TROW];
     double G[MC_T];
     float ik[MC_T], ek[MC_T], wk[MC_T], eg[MC_T];
     float c[MC_T];        // e^G * q_scale / |q|
     float qs[NW][MC_T];   // shares of |q|^2
   };
-  __shared__ Shared sm;
+  __shared__ __align__(16) Shared sm;
 
   const int seg = blockIdx.x, h = blockIdx.y;
   const int n = A.seg_len[seg];
@@ -241,7 +245,7 @@ __global__ __launch_bounds__(NW * WAVE_SIZE) void delta_chunk_scan_kernel(
   const int col = (wave & 3) * 16 + li;  // the state column this lane holds
   const uint16_t* q = (const uint16_t*)A.q + (h / A.rep) * D;
   const uint16_t* k = (const uint16_t*)A.k + (h / A.rep) * D;
-  const uint16_t* v = (const uint16_t*)A.v + h * Dv + c0 + col;
+  const uint16_t* v = (const uint16_t*)A.v + h * Dv + (active ? c0 : 0);
   const DeltaChunk* ch = scratch + delta_chunk_slot(r0, 0, seg) * H + h;
 
   // ---- state row: [head][block][entry][column * split + key lane] ----------------------
@@ -259,27 +263,36 @@ __global__ __launch_bounds__(NW * WAVE_SIZE) void delta_chunk_scan_kernel(
     }
   }
   // the blocks above the diagonal are never written: zero for the whole walk
-  for (int e = tid; e < 2 * MC_T * MC_TP / 8; e += NW * WAVE_SIZE) {
+  for (int e = tid; e < 2 * MC_T * TROW / 8; e += NW * WAVE_SIZE) {
     const u16x8 z = {0, 0, 0, 0, 0, 0, 0, 0};
     reinterpret_cast<u16x8*>(&sm.t[0][0][0])[e] = z;
     reinterpret_cast<u16x8*>(&sm.p[0][0][0])[e] = z;
   }
 
-  // a thread stages token `lane`, 16-byte chunks wave, wave + NW, ...
+  // A thread stages token `lane`, 16-byte chunks wave, wave + NW, ...  Rows past
+  // the portion's end read its last token instead: their write strength and
+  // their weight in the state are zero and their outputs are not stored.
   u16x8 qr[NCH], kr[NCH], tr[NT];
   uint16_t vr[16];
   double Gr = 0.0;
   float sr[4] = {0.f, 0.f, 0.f, 0.f};
   const u16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
+  const int q_stride = (int)A.q_stride, k_stride = (int)A.k_stride, v_stride = (int)A.v_stride;
+  const int q_off = lane * q_stride, k_off = lane * k_stride;
+  const bool col_ok = col < ncol;
+  const int v_off = lg * 4 * v_stride + (col_ok ? col : 0);
   auto fetch = [&](int t0) __attribute__((always_inline)) {
-    const bool ok = t0 + lane < n;
-    const long r = r0 + t0 + lane;
+    const uint16_t* qb = q + (r0 + t0) * A.q_stride;
+    const uint16_t* kb = k + (r0 + t0) * A.k_stride;
+    const int last = n - 1 - t0;
+    const int qo = last < MC_T - 1 ? min(lane, last) * q_stride : q_off;
+    const int ko = last < MC_T - 1 ? min(lane, last) * k_stride : k_off;
 #pragma unroll
     for (int j = 0; j < NCH; ++j) {
       const int d = (wave + NW * j) * 8;
-      const bool in = ok && d < D;
-      qr[j] = in ? mc_ld16(q + r * A.q_stride + d) : zero8;
-      kr[j] = in ? mc_ld16(k + r * A.k_stride + d) : zero8;
+      const bool in = d < D;  // uniform over the wave
+      qr[j] = in ? mc_ld16(qb + qo + d) : zero8;
+      kr[j] = in ? mc_ld16(kb + ko + d) : zero8;
     }
     const DeltaChunk* c = ch + (long)(t0 / MC_T) * H;
 #pragma unroll
@@ -287,15 +300,7 @@ __global__ __launch_bounds__(NW * WAVE_SIZE) void delta_chunk_scan_kernel(
       const int e = tid + j * NW * WAVE_SIZE;
       const int t = (e / 8) % MC_T, s0 = (e % 8) * 8;
       const uint16_t* src = e < MC_T * MC_T / 8 ? &c->t_hi[t][s0] : &c->t_lo[t][s0];
-      tr[j] = (s0 / 16 <= t / 16) ? mc_ld16(src) : zero8;
-    }
-#pragma unroll
-    for (int tt = 0; tt < 4; ++tt) {
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int t = t0 + tt * 16 + lg * 4 + i;
-        vr[tt * 4 + i] = (t < n && col < ncol) ? v[(r0 + t) * A.v_stride] : (uint16_t)0;
-      }
+      if (s0 / 16 <= t / 16) tr[j] = mc_ld16(src);
     }
     if (tid < MC_T) {
       Gr = c->G[tid];
@@ -305,7 +310,21 @@ __global__ __launch_bounds__(NW * WAVE_SIZE) void delta_chunk_scan_kernel(
       sr[3] = c->eg[tid];
     }
   };
+  // values of token tt * 16 + lg * 4 + i, column col
+  auto fetch_v = [&](int t0) __attribute__((always_inline)) {
+    const uint16_t* vb = v + (r0 + t0) * A.v_stride;
+    const int last = n - 1 - t0;
+    if (last >= MC_T - 1) {
+#pragma unroll
+      for (int e = 0; e < 16; ++e) vr[e] = vb[v_off + ((e >> 2) * 16 + (e & 3)) * v_stride];
+    } else {
+#pragma unroll
+      for (int e = 0; e < 16; ++e)
+        vr[e] = vb[min((e >> 2) * 16 + lg * 4 + (e & 3), last) * v_stride + (col_ok ? col : 0)];
+    }
+  };
   fetch(0);
+  fetch_v(0);
 
 #pragma nounroll
   for (int t0 = 0; t0 < n; t0 += MC_T) {
@@ -317,8 +336,8 @@ __global__ __launch_bounds__(NW * WAVE_SIZE) void delta_chunk_scan_kernel(
     for (int j = 0; j < NCH; ++j) {
       const int d = (wave + NW * j) * 8;
       if (d < DP) {
-        *reinterpret_cast<u16x8*>(&sm.q[lane][d]) = qr[j];
-        *reinterpret_cast<u16x8*>(&sm.k[lane][d]) = kr[j];
+        mc_st8x2(&sm.q[lane][d], qr[j]);
+        mc_st8x2(&sm.k[lane][d], kr[j]);
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
           sm.kt[d + e][lane] = kr[j][e];
@@ -332,7 +351,7 @@ __global__ __launch_bounds__(NW * WAVE_SIZE) void delta_chunk_scan_kernel(
     for (int j = 0; j < NT; ++j) {
       const int e = tid + j * NW * WAVE_SIZE;
       const int half = e / (MC_T * MC_T / 8), t = (e / 8) % MC_T, s0 = (e % 8) * 8;
-      if (s0 / 16 <= t / 16) *reinterpret_cast<u16x8*>(&sm.t[half][t][s0]) = tr[j];
+      if (s0 / 16 <= t / 16) mc_st8x2(&sm.t[half][t][s0], tr[j]);
     }
     if (tid < MC_T) {
       sm.G[tid] = Gr;
@@ -341,12 +360,6 @@ __global__ __launch_bounds__(NW * WAVE_SIZE) void delta_chunk_scan_kernel(
       sm.wk[tid] = sr[2];
       sm.eg[tid] = sr[3];
     }
-    // this chunk's values, token tt * 16 + lg * 4 + r of column col
-    f32x4 R[4];
-#pragma unroll
-    for (int tt = 0; tt < 4; ++tt)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) R[tt][i] = bf16_to_f32(vr[tt * 4 + i]);
     __syncthreads();
     if (t0 + MC_T < n) fetch(t0 + MC_T);
 
@@ -364,95 +377,72 @@ __global__ __launch_bounds__(NW * WAVE_SIZE) void delta_chunk_scan_kernel(
 #pragma unroll
         for (int kb = 0; kb < KB; ++kb) {
           const int d = kb * 32 + lg * 8;
-          acc = mc_mfma(mc_ld16(&sm.k[st * 16 + li][d]), mc_ld16(&sm.q[t][d]), acc);
+          const uint16_t *kp = &sm.k[st * 16 + li][d], *qp = &sm.q[t][d];
+          acc = mc_mfma(mc_ld8x2(kp, kp + 4), mc_ld8x2(qp, qp + 4), acc);
         }
-        u16x4 hi, lo;
+        f32x4 p;
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int s = st * 16 + lg * 4 + r;
-          float p = 0.f;
-          if (s <= t) p = acc[r] * iq * sm.ik[s] * __expf((float)(Gt - sm.G[s]));
-          uint16_t a, b;
-          mc_split(p, a, b);
-          hi[r] = a;
-          lo[r] = b;
+          p[r] = s <= t ? acc[r] * iq * sm.ik[s] * __expf((float)(Gt - sm.G[s])) : 0.f;
         }
-        *reinterpret_cast<u16x4*>(&sm.p[0][t][st * 16 + lg * 4]) = hi;
-        *reinterpret_cast<u16x4*>(&sm.p[1][t][st * 16 + lg * 4]) = lo;
+        uint32_t h0, h1, l0, l1;
+        mc_split2(p[0], p[1], h0, l0);
+        mc_split2(p[2], p[3], h1, l1);
+        *reinterpret_cast<u32x2*>(&sm.p[0][t][st * 16 + lg * 4]) = u32x2{h0, h1};
+        *reinterpret_cast<u32x2*>(&sm.p[1][t][st * 16 + lg * 4]) = u32x2{l0, l1};
       }
     }
     f32x4 o[4];
-    u16x8 uh[2], ul[2], wh[2], wl[2];
+    u32x4 uh[2], ul[2], wh[2], wl[2];
     if (active) {
-      u16x8 sh[KB], sl[KB];
+      // ---- the chunk's starting state with all keys and all queries ---------------------------
+      f32x4 x[4];
+#pragma unroll
+      for (int tt = 0; tt < 4; ++tt) x[tt] = o[tt] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int u = 0; u < KB; ++u) {
+        u32x4 sh, sl;
+        mc_split4(S[2 * u], 0, sh, sl);
+        mc_split4(S[2 * u + 1], 1, sh, sl);
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          uint16_t a, b;
-          mc_split(S[2 * u][r], a, b);
-          sh[u][r] = a;
-          sl[u][r] = b;
-          mc_split(S[2 * u + 1][r], a, b);
-          sh[u][4 + r] = a;
-          sl[u][4 + r] = b;
+        for (int tt = 0; tt < 4; ++tt) {
+          const uint16_t* kp = &sm.k[tt * 16 + li][u * 32 + lg * 4];
+          const uint16_t* qp = &sm.q[tt * 16 + li][u * 32 + lg * 4];
+          const u16x8 a = mc_ld8x2(kp, kp + 16), b = mc_ld8x2(qp, qp + 16);
+          x[tt] = mc_mfma(a, sh, x[tt]);
+          o[tt] = mc_mfma(sh, b, o[tt]);
+          x[tt] = mc_mfma(a, sl, x[tt]);
+          o[tt] = mc_mfma(sl, b, o[tt]);
         }
       }
       // ---- right-hand sides: v - e^G S^T k ---------------------------------------------------
-      u16x8 rh[2], rl[2];
+      u32x4 rh[2], rl[2];
 #pragma unroll
       for (int tt = 0; tt < 4; ++tt) {
-        f32x4 x = {0.f, 0.f, 0.f, 0.f};
-        const uint16_t* kp = &sm.k[tt * 16 + li][lg * 4];
+        const f32x4 ek = *reinterpret_cast<const f32x4*>(&sm.ek[tt * 16 + lg * 4]);
+        f32x4 val;
 #pragma unroll
-        for (int u = 0; u < KB; ++u) {
-          const u16x8 a = mc_ld8x2(kp + u * 32, kp + u * 32 + 16);
-          x = mc_mfma(a, sh[u], x);
-          x = mc_mfma(a, sl[u], x);
-        }
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          uint16_t a, b;
-          mc_split(R[tt][r] - sm.ek[tt * 16 + lg * 4 + r] * x[r], a, b);
-          rh[tt / 2][(tt & 1) * 4 + r] = a;
-          rl[tt / 2][(tt & 1) * 4 + r] = b;
-        }
+        for (int i = 0; i < 4; ++i) val[i] = col_ok ? bf16_to_f32(vr[tt * 4 + i]) : 0.f;
+        mc_split4(val - ek * x[tt], tt & 1, rh[tt / 2], rl[tt / 2]);
       }
+      if (t0 + MC_T < n) fetch_v(t0 + MC_T);
       // ---- corrections u = inverse * right-hand sides ----------------------------------------
 #pragma unroll
       for (int tt = 0; tt < 4; ++tt) {
-        f32x4 x = {0.f, 0.f, 0.f, 0.f};
+        f32x4 c = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int u = 0; u <= tt / 2; ++u) {
           const uint16_t* th = &sm.t[0][tt * 16 + li][u * 32 + lg * 4];
           const uint16_t* tl = &sm.t[1][tt * 16 + li][u * 32 + lg * 4];
           const u16x8 a = mc_ld8x2(th, th + 16);
-          x = mc_mfma(a, rh[u], x);
-          x = mc_mfma(a, rl[u], x);
-          x = mc_mfma(mc_ld8x2(tl, tl + 16), rh[u], x);
+          c = mc_mfma(a, rh[u], c);
+          c = mc_mfma(a, rl[u], c);
+          c = mc_mfma(mc_ld8x2(tl, tl + 16), rh[u], c);
         }
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          uint16_t a, b;
-          mc_split(x[r], a, b);
-          uh[tt / 2][(tt & 1) * 4 + r] = a;
-          ul[tt / 2][(tt & 1) * 4 + r] = b;
-          mc_split(x[r] * sm.wk[tt * 16 + lg * 4 + r], a, b);
-          wh[tt / 2][(tt & 1) * 4 + r] = a;
-          wl[tt / 2][(tt & 1) * 4 + r] = b;
-        }
-      }
-      // ---- the chunk's starting state with all queries ------------------------------------------
-#pragma unroll
-      for (int tt = 0; tt < 4; ++tt) {
-        o[tt] = f32x4{0.f, 0.f, 0.f, 0.f};
-        const uint16_t* qp = &sm.q[tt * 16 + li][lg * 4];
-#pragma unroll
-        for (int u = 0; u < KB; ++u) {
-          const u16x8 b = mc_ld8x2(qp + u * 32, qp + u * 32 + 16);
-          o[tt] = mc_mfma(sh[u], b, o[tt]);
-          o[tt] = mc_mfma(sl[u], b, o[tt]);
-        }
+        const f32x4 wk = *reinterpret_cast<const f32x4*>(&sm.wk[tt * 16 + lg * 4]);
+        mc_split4(c, tt & 1, uh[tt / 2], ul[tt / 2]);
+        mc_split4(c * wk, tt & 1, wh[tt / 2], wl[tt / 2]);
       }
     }
     __syncthreads();
@@ -504,7 +494,10 @@ __global__ __launch_bounds__(NW * WAVE_SIZE) void delta_chunk_scan_kernel(
 }
 
 bool ms_delta_chunks_served(const MsArgs& a) {
-  return a.D % 8 == 0 && a.Dv % 8 == 0 && a.D <= 256 && a.q_stride % 8 == 0 &&
+  // offsets inside a chunk are 32-bit
+  const long lim = 2147483647L / MC_T;
+  return a.q_stride <= lim && a.k_stride <= lim && a.v_stride <= lim && a.D % 8 == 0 &&
+         a.Dv % 8 == 0 && a.D <= 256 && a.q_stride % 8 == 0 &&
          a.k_stride % 8 == 0 && aligned16(a.q) && aligned16(a.k) && aligned16(a.out);
 }
 
@@ -512,12 +505,16 @@ void ms_delta_chunks_launch(const MsArgs& a, int S, int max_seg_len, void* scrat
                             hipStream_t st) {
   DeltaChunk* sc = (DeltaChunk*)scratch;
   const dim3 gi((max_seg_len + MC_T - 1) / MC_T, S, a.H);
+  // two value blocks per workgroup share the staged operands where the
+  // registers of eight waves hold the state
 #define LIG_DC(DP)                                                                            \
   do {                                                                                        \
     hipLaunchKernelGGL(delta_chunk_inverse_kernel<DP>, gi, dim3(DI_THREADS), 0, st, a, sc);   \
+    constexpr int NW = DP <= 128 ? 8 : 4;                                                     \
     if (a.NB > 1)                                                                             \
-      hipLaunchKernelGGL((delta_chunk_scan_kernel<DP, 8>), dim3(S, a.H, (a.NB + 1) / 2),      \
-                         dim3(8 * WAVE_SIZE), 0, st, a, sc);                                  \
+      hipLaunchKernelGGL((delta_chunk_scan_kernel<DP, NW>),                                   \
+                         dim3(S, a.H, (a.NB + NW / 4 - 1) / (NW / 4)), dim3(NW * WAVE_SIZE),  \
+                         0, st, a, sc);                                                       \
     else                                                                                      \
       hipLaunchKernelGGL((delta_chunk_scan_kernel<DP, 4>), dim3(S, a.H, 1),                   \
                          dim3(4 * WAVE_SIZE), 0, st, a, sc);                                  \

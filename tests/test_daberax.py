@@ -469,9 +469,8 @@ def test_sizes_of_the_mfma_kernels(model_c, device, dtype):
 @pytest.mark.parametrize("which", ["a", "c"])
 def test_decode_graphs_replay_like_eager(model_a, model_c, dtype, which):
     """Decode-only steps replay captured hipGraphs (static per-sequence
-    tables, state slots filled per step).  Many
-    replays with eager prefill steps of later requests in between; every
-    generated token is checked."""
+    tables, state slots filled per step).  Many replays with eager prefill
+    steps of later requests in between; every generated token is checked."""
     path, W = model_a if which == "a" else model_c
     cfg = CFG_A if which == "a" else CFG_C
     eng = make_engine(path, "cuda:0", dtype, budget=32, enforce_eager=False)
@@ -489,6 +488,34 @@ def test_decode_graphs_replay_like_eager(model_a, model_c, dtype, which):
     for seq, prompt in zip(seqs, prompts):
         assert seq.is_finished()
         assert_greedy_follows_oracle(cfg, W, prompt, seq.output_token_ids, margin)
+
+
+@pytest.mark.gpu
+def test_an_engine_captures_while_a_dropped_one_awaits_collection(model_c):
+    """Graphs of a dropped engine must not be destroyed inside another
+    engine's capture, however eagerly the collector runs."""
+    import gc
+
+    path, _ = model_c
+    prompt = tokens_for(CFG_C, 9, 1)
+    outs = []
+    before = gc.get_threshold()
+    gc.set_threshold(5, 1, 1)
+    try:
+        for _ in range(2):
+            gc.disable()  # the dropped engine's cycles stay until the next capture
+            eng = make_engine(path, "cuda:0", torch.bfloat16, enforce_eager=False)
+            gc.enable()
+            seq = eng.add_request(prompt, SamplingParams(max_new_tokens=4))
+            eng.generate_all(max_steps=20)
+            assert eng.runner.graph_runner.graphs and gc.isenabled()
+            outs.append(seq.output_token_ids)
+            gc.disable()
+            del eng, seq
+    finally:
+        gc.enable()
+        gc.set_threshold(*before)
+    assert outs[0] == outs[1]
 
 
 def test_served_through_the_pool_and_front_door(tmp_path):
