@@ -70,8 +70,10 @@ extern "C" int lig_small_projection(float* out, const void* h, const void* w, in
   hipLaunchKernelGGL(small_projection_kernel<NT>, dim3(rows, (N + NT * 16 - 1) / (NT * 16)),   \
                      dim3(SP_WAVES * WAVE_SIZE), 0, s, out, (const uint16_t*)h,                \
                      (const uint16_t*)w, R, N, C)
-  if (N <= 16) LIG_SP(1);
-  else if (N <= 32) LIG_SP(2);
+  // few rows (decode steps): narrower column tiles, so that a wave has fewer
+  // loads in its chain and more workgroups share the columns
+  if (N <= 16 || (long)rows * ((N + 31) / 32) < 256) LIG_SP(1);
+  else if (N <= 32 || (long)rows * ((N + 63) / 64) < 256) LIG_SP(2);
   else LIG_SP(4);
 #undef LIG_SP
   return 0;
